@@ -3,8 +3,8 @@
 ``get_module``, loader.py:23-54).
 
 The reference globs ``lib/*.so`` and imports each file as a pybind module. The
-MI355X backend is one plain C-ABI library (no ``PyInit_*``), so the registry
-binds it with ctypes and exposes, per kernel name, an adapter object carrying
+MI355X backend is two plain C-ABI libraries (no ``PyInit_*``), so the registry
+binds them with ctypes and exposes, per kernel name, an adapter object carrying
 the callables the pybind module of that name carries. A kernel whose library is
 absent is reported unavailable (``False`` / ``None``), never by an exception at
 import, exactly as the reference does (loader.py:36-44).
@@ -15,7 +15,7 @@ from __future__ import annotations
 import logging
 from types import SimpleNamespace
 
-from astrai_amd.extension import _cabi
+from astrai_amd.extension import _cabi, _mix
 
 logger = logging.getLogger(__name__)
 
@@ -86,6 +86,27 @@ def _rotary_emb_module() -> SimpleNamespace:
     return SimpleNamespace(rotary_emb=_cabi.rotary_emb)
 
 
+# the mechanisms of libastrai_mix.so (none of them exists in the reference)
+def _latent_attention_module() -> SimpleNamespace:
+    return SimpleNamespace(latent_append=_mix.latent_append, latent_prefill=_mix.latent_prefill,
+                           latent_rows=_mix.latent_rows)
+
+
+def _lightning_attention_module() -> SimpleNamespace:
+    return SimpleNamespace(lightning=_mix.lightning, decay_powers=_mix.decay_powers)
+
+
+def _residual_rows_module() -> SimpleNamespace:
+    return SimpleNamespace(residual_norm=_mix.residual_norm, embed_norm=_mix.embed_norm, silu_mul=_mix.silu_mul,
+                           gated_rms_norm=_mix.gated_rms_norm)
+
+
+_MIX_FACTORIES = {
+    "latent_attention": _latent_attention_module,
+    "lightning_attention": _lightning_attention_module,
+    "residual_rows": _residual_rows_module,
+}
+
 _FACTORIES = {
     "attn_decode": _attn_decode_module,
     "attn_prefill": _attn_prefill_module,
@@ -97,7 +118,7 @@ _FACTORIES = {
     "fp8_block_mm": _fp8_block_mm_module,
 }
 
-KERNEL_NAMES = sorted(_FACTORIES)
+KERNEL_NAMES = sorted([*_FACTORIES, *_MIX_FACTORIES])
 
 _available: dict[str, bool] = {}
 _modules: dict[str, object] = {}
@@ -105,9 +126,13 @@ _modules: dict[str, object] = {}
 _loaded = _cabi.load() is not None
 if not _loaded:
     logger.debug("libastrai_w8a8.so unavailable: %s", _cabi.load_error())
-for _name in KERNEL_NAMES:
-    _available[_name] = _loaded
-    _modules[_name] = _FACTORIES[_name]() if _loaded else None
+_mix_loaded = _mix.load() is not None
+if not _mix_loaded:
+    logger.debug("libastrai_mix.so unavailable: %s", _mix.load_error())
+for _factories, _ok in ((_FACTORIES, _loaded), (_MIX_FACTORIES, _mix_loaded)):
+    for _name, _factory in _factories.items():
+        _available[_name] = _ok
+        _modules[_name] = _factory() if _ok else None
 
 
 def is_available(name: str) -> bool:

@@ -33,6 +33,26 @@ _WEIGHTS_FILE = "model.safetensors"
 SCHEME = "int8_w8a8_per_channel"
 
 
+@torch.no_grad()
+def load_checkpoint(model_dir: str, device="cuda", dtype: torch.dtype = torch.bfloat16) -> torch.nn.Module:
+    """Build the model that ``model_dir/config.json`` names (``registry``) on ``device`` in ``dtype`` with
+    the weights of ``model.safetensors``. An int8 checkpoint goes to :func:`load_int8_checkpoint`."""
+    from astrai_amd.model.registry import architecture_of
+
+    path = Path(model_dir)
+    meta = json.loads((path / _META_FILE).read_text()) if (path / _META_FILE).exists() else {}
+    if meta.get("quantization", {}).get("scheme") == SCHEME:
+        if dtype != torch.bfloat16:
+            raise ValueError(f"{model_dir} is an {SCHEME} checkpoint: bfloat16 only")
+        return load_int8_checkpoint(model_dir, device)
+    config = json.loads((path / _CONFIG_FILE).read_text())
+    arch = architecture_of(config)
+    tensors = st.load_file(str(path / _WEIGHTS_FILE))  # safetensors: data only, nothing executed
+    with torch.device(device):
+        model = arch.model_class(arch.make_config(config)).to(dtype).eval()
+    return model.load_tensors(tensors)
+
+
 def _linear_names(model: AutoRegressiveLM):
     return [name for name, mod in model.named_modules() if isinstance(mod, Linear)]
 
@@ -94,10 +114,7 @@ def load_int8_checkpoint(save_dir: str, device="cuda", fuse: bool = True) -> Aut
             plain[base] = (wq.float() * sw.reshape(-1, 1)).to(torch.bfloat16)
         elif not name.endswith(".weight_scale"):
             plain[name] = t.to(device)
-    missing, unexpected = model.load_state_dict(plain, strict=False)
-    missing = [m for m in missing if not (cfg.tie_word_embeddings and m == "lm_head.weight")]
-    if missing or unexpected:
-        raise ValueError(f"checkpoint does not match the model: missing {missing}, unexpected {unexpected}")
+    model.load_tensors(plain)
     params = dict(model.named_parameters())
     state = w8a8.int8_state()
     for base, (wq, sw) in quantized.items():

@@ -26,6 +26,7 @@ per element is that of the modular path (concatenating per-channel quantized row
 changes no row; the fused producers round where the separate ops round).
 """
 
+import math
 from dataclasses import dataclass
 from types import SimpleNamespace
 from typing import Dict, Optional
@@ -34,6 +35,8 @@ import torch
 import torch.nn as nn
 import torch.nn.functional as F
 from torch import Tensor
+
+from astrai_amd.model.cache import StepCache
 
 
 @dataclass
@@ -102,6 +105,25 @@ def get_rotary_emb(dim: int, max_len: int, base: float = 10000.0) -> Tensor:
     return torch.stack([torch.cos(freqs), torch.sin(freqs)], dim=-1)
 
 
+def rotary_table(freqs: Tensor, max_len: int, magnitude: float = 1.0) -> Tensor:
+    """``[max_len, len(freqs), 2]`` fp32 table of ``magnitude`` times (cos, sin) of position times frequency;
+    everything up to the last rounding in fp64."""
+    ang = torch.outer(torch.arange(max_len, dtype=torch.float64, device=freqs.device), freqs.double())
+    return (torch.stack([torch.cos(ang), torch.sin(ang)], dim=-1) * magnitude).float()
+
+
+def yarn_frequencies(dims: int, base: float, factor: float, original: float, fast: float, slow: float) -> Tensor:
+    """YaRN-scaled rotary frequencies, ``[dims / 2]`` fp64: pairs that turn more than ``fast`` times over the
+    ``original`` context keep ``base^(-2i/dims)``, those that turn fewer than ``slow`` times get ``1/factor`` of
+    it, with a linear ramp over the pair index in between."""
+    i = torch.arange(dims // 2, dtype=torch.float64)
+    freqs = base ** (-2.0 * i / dims)
+    lo, hi = (dims * math.log(original / (2 * math.pi * turns)) / (2 * math.log(base)) for turns in (fast, slow))
+    lo, hi = max(math.floor(lo), 0), min(math.ceil(hi), dims - 1)
+    ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0, 1)
+    return freqs / factor * ramp + freqs * (1 - ramp)
+
+
 def ntk_base(base: float, dim: int, factor: float) -> float:
     """NTK-aware stretching of the rotary base (components/rope.py:27-28)."""
     return base * (factor ** (dim / (dim - 2)))
@@ -136,15 +158,15 @@ def repeat_kv(x: Tensor, n_rep: int) -> Tensor:
     return x.unsqueeze(2).expand(b, h, n_rep, s, d).reshape(b, h * n_rep, s, d)
 
 
-class DenseKVCache:
+class DenseKVCache(StepCache):
     """``k``/``v``: ``[layers, batch, kv_heads, max_len, head_dim]``."""
 
     def __init__(self, config: AutoRegressiveLMConfig, batch: int, max_len: int, device, dtype):
+        super().__init__(batch, max_len, device)
         hd = config.hidden_size // config.num_attention_heads
         shape = (config.num_hidden_layers, batch, config.num_key_value_heads, max_len, hd)
         self.k = torch.zeros(shape, device=device, dtype=dtype)
         self.v = torch.zeros(shape, device=device, dtype=dtype)
-        self.max_len = max_len
 
 
 class GQA(nn.Module):
@@ -343,18 +365,33 @@ class AutoRegressiveLM(nn.Module):
         self.apply(lambda m: m.reset_parameters() if hasattr(m, "reset_parameters") else None)
         self.fused_int8 = None  # set by fuse_int8_weights
 
+    @torch.no_grad()
+    def load_tensors(self, tensors: Dict[str, Tensor]) -> "AutoRegressiveLM":
+        """Take every weight from ``tensors``; a missing or unknown one raises (a tied head may be absent)."""
+        missing, unexpected = self.load_state_dict(tensors, strict=False)
+        missing = [m for m in missing if not (self.config.tie_word_embeddings and m == "lm_head.weight")]
+        if missing or unexpected:
+            raise ValueError(f"checkpoint does not match the model: missing {missing}, unexpected {unexpected}")
+        return self
+
+    def new_cache(self, batch: int, max_len: int) -> DenseKVCache:
+        w = self.embed_tokens.weight
+        return DenseKVCache(self.config, batch, max_len, w.device, w.dtype)
+
     def forward(self, input_ids: Tensor, kv_cache: Optional[DenseKVCache] = None,
-                positions: Optional[Tensor] = None) -> Dict[str, Tensor]:
+                positions: Optional[Tensor] = None, logits_at: Optional[Tensor] = None) -> Dict[str, Tensor]:
         """``input_ids [batch, seq]``. Without a cache: causal forward over the block.
         With a cache: the block's tokens sit at ``positions`` (``[seq]`` int64, on the
-        device), keys/values are written there and every query attends to cache
-        entries at positions <= its own."""
+        device; by default those after the tokens the cache holds), keys/values are written
+        there and every query attends to cache entries at positions <= its own.
+        ``logits_at``: indices into the block; only these tokens' logits are returned."""
         if input_ids.ndim != 2:
             raise ValueError("input_ids must be [batch, seq_len]")
         b, s = input_ids.shape
         x = self.embed_tokens(input_ids)
         if positions is None:
-            positions = torch.arange(s, device=input_ids.device)
+            positions = (torch.arange(s, device=input_ids.device) if kv_cache is None
+                         else kv_cache.next_positions(s))
         rotary = self.freqs_cis.index_select(0, positions).unsqueeze(0).float()
         key_mask = None
         if kv_cache is not None:
@@ -364,12 +401,16 @@ class AutoRegressiveLM(nn.Module):
             from astrai_amd.extension import _cabi
             for layer in self.layers:
                 x = layer._forward_fused_int8(x, rotary, kv_cache, positions, key_mask)
+            if logits_at is not None:
+                s, x = logits_at.numel(), x.index_select(1, logits_at)
             hq, sh, _, hidden = _cabi.add_rmsnorm_quantize_int8(x, self.norm.weight, self.norm.norm_eps,
                                                                 None, True)
             logits = _cabi.mm_int8(hq, self.fused_int8.wlm, sh, self.fused_int8.slm).reshape(b, s, -1)
             return {"logits": logits, "hidden_states": hidden}
         for layer in self.layers:
             x = layer(x, rotary, kv_cache, positions, key_mask)
+        if logits_at is not None:
+            x = x.index_select(1, logits_at)
         hidden = self.norm(x)
         return {"logits": self.lm_head(hidden), "hidden_states": hidden}
 
@@ -429,17 +470,17 @@ def unfuse_int8_weights(model: AutoRegressiveLM) -> None:
 
 
 @torch.no_grad()
-def greedy_generate(model: AutoRegressiveLM, prompt_ids: Tensor, steps: int,
+def greedy_generate(model: nn.Module, prompt_ids: Tensor, steps: int,
                     use_graph: bool = False, warmup_steps: int = 2) -> Tensor:
-    """Prefill ``prompt_ids [batch, prompt_len]`` then ``steps`` greedy (argmax) decode
+    """For any registered model (its ``new_cache`` and forward): prefill ``prompt_ids [batch, prompt_len]`` then ``steps`` greedy (argmax) decode
     steps; returns the generated ids ``[batch, steps]``. With ``use_graph`` the decode
     step is captured after ``warmup_steps`` eager steps and replayed
     (the reference's warm -> capture -> replay pattern, inference/runtime/graph.py:86-100)."""
     b, p = prompt_ids.shape
     dev = prompt_ids.device
-    dtype = model.embed_tokens.weight.dtype
-    cache = DenseKVCache(model.config, b, p + steps, dev, dtype)
+    cache = model.new_cache(b, p + steps)
     logits = model(prompt_ids, cache, torch.arange(p, device=dev))["logits"]
+    cache.advance(p)
     tok = logits[:, -1].argmax(-1)
     out = torch.empty(b, steps, dtype=torch.long, device=dev)
     cur = tok.clone().reshape(b, 1)
@@ -466,6 +507,7 @@ def greedy_generate(model: AutoRegressiveLM, prompt_ids: Tensor, steps: int,
             nxt = nxt_static
         else:
             nxt = step()
+        cache.advance(1)
         cur.copy_(nxt.reshape(b, 1))
         pos.add_(1)
     return out
