@@ -9,6 +9,8 @@
 
 #include "mix_launchers.h"
 
+static_assert(astrai_mix::kMaxSplit == ASTRAI_MIX_MAX_SPLIT && astrai_mix::kLightningChunk == ASTRAI_MIX_LIGHTNING_CHUNK);
+
 namespace {
 
 using namespace astrai_mix;
@@ -182,8 +184,8 @@ int astrai_mix_gated_rms_norm(const void* o, const void* g, int64_t ldg, const f
 }
 
 int astrai_mix_latent_append(void* proj, int64_t ld, int64_t dkv_off, const float* rot, int64_t rot_rows, int64_t half,
-                             const int64_t* positions, const float* norm_w, void* cache, int64_t batch, int64_t seq,
-                             int64_t max_len, int64_t heads, int64_t dn, int64_t dr, int64_t rp, int64_t kv_rank,
+                             const int64_t* positions, const float* norm_w, void* cache, const void* w_uk_t, void* q_abs,
+                             int64_t batch, int64_t seq, int64_t max_len, int64_t heads, int64_t dn, int64_t dr, int64_t rp, int64_t kv_rank,
                              float eps, int dtype, void* stream) {
     MIX_TRY(check_dtype("latent_append", dtype));
     MIX_TRY(check_ptrs("latent_append", (const void*)proj, (const void*)rot));
@@ -196,6 +198,12 @@ int astrai_mix_latent_append(void* proj, int64_t ld, int64_t dkv_off, const floa
         kv_rank > rp || rot_rows <= 0 || heads * half > kMaxInt)
         return fail(ASTRAI_MIX_BAD_ARG, "latent_append: bad columns (dkv_off %lld, half %lld, kv_rank %lld)",
                     (long long)dkv_off, (long long)half, (long long)kv_rank);
+    if (q_abs) {
+        MIX_TRY(check_ptrs("latent_append", w_uk_t, (const void*)q_abs));
+        if (dtype != ASTRAI_MIX_BF16 || batch * seq > (1 << 20) || heads * (rp / 32) > (1 << 20) ||
+            batch * seq * heads * ((rp + 63) / 64) > kMaxInt)
+            return fail(ASTRAI_MIX_UNSUPPORTED, "latent_append: absorbed queries are bf16, for %lld tokens at most", 1LL << 20);
+    }
     LatentAppendArgs a;
     a.proj = proj;
     a.ld = ld;
@@ -204,6 +212,8 @@ int astrai_mix_latent_append(void* proj, int64_t ld, int64_t dkv_off, const floa
     a.positions = positions;
     a.norm_w = norm_w;
     a.cache = cache;
+    a.w_uk_t = w_uk_t;
+    a.q_abs = q_abs;
     a.tokens = batch * seq;
     a.rot_rows = rot_rows;
     a.seq = (int)seq;
@@ -231,8 +241,8 @@ int astrai_mix_latent_prefill(const void* proj, int64_t ld, int64_t g_off, const
     if (g_off < 0 || g_off + heads > ld) return fail(ASTRAI_MIX_BAD_ARG, "latent_prefill: bad gate column");
     const LatentDims d = dims(heads, dn, dr, rp, vp, window, scale);
     if (!latent_prefill_supported(d) || ((seq + 127) / 128) * batch * heads > kMaxInt)
-        return fail(ASTRAI_MIX_UNSUPPORTED, "latent_prefill: head sizes %lld + %lld, value %lld (at most 256, 128)",
-                    (long long)dn, (long long)dr, (long long)vp);
+        return fail(ASTRAI_MIX_UNSUPPORTED, "latent_prefill: head sizes %lld + %lld, value %lld (at most 128, 64, 128) or scale %g",
+                    (long long)dn, (long long)dr, (long long)vp, (double)scale);
     LatentPrefillArgs a;
     a.proj = proj;
     a.ld = ld;
@@ -254,21 +264,22 @@ int64_t astrai_mix_latent_rows_workspace_floats(int64_t tokens, int64_t heads, i
     return latent_rows_workspace_floats(dims(heads, 32, 32, rp, 32, 1, 1.0f), tokens, (int)nsplit);
 }
 
-int astrai_mix_latent_rows(const void* proj, int64_t ld, int64_t g_off, const void* w_ukv, const void* w_uk_t,
-                           const void* cache, const int64_t* positions, void* q_abs, float* ws, void* out,
+int astrai_mix_latent_rows(const void* proj, int64_t ld, int64_t g_off, const void* w_ukv, const void* cache,
+                           const int64_t* positions, void* q_abs, float* ws, void* out,
                            int64_t batch, int64_t seq, int64_t max_len, int64_t heads, int64_t dn, int64_t dr,
                            int64_t rp, int64_t vp, int64_t window, float scale, int64_t nsplit, void* stream) {
-    MIX_TRY(check_ptrs("latent_rows", proj, w_ukv, w_uk_t, cache, (const void*)q_abs, (const void*)ws, (const void*)out));
+    MIX_TRY(check_ptrs("latent_rows", proj, w_ukv, cache, (const void*)q_abs, (const void*)ws, (const void*)out));
     if (!positions) return fail(ASTRAI_MIX_BAD_ARG, "latent_rows: null pointer");
     MIX_TRY(check_heads("latent_rows", heads, dn, dr, rp, vp));
     MIX_TRY(check_block("latent_rows", batch, seq, max_len, ld, heads * (dn + dr)));
-    if (window <= 0 || g_off < 0 || g_off + heads > ld || nsplit < 1 || nsplit > ASTRAI_MIX_MAX_SPLIT)
+    if (window <= 0 || g_off < 0 || g_off + heads > ld || nsplit < 1 || nsplit > kMaxSplit)
         return fail(ASTRAI_MIX_BAD_ARG, "latent_rows: bad window, gate column or nsplit %lld", (long long)nsplit);
     const LatentDims d = dims(heads, dn, dr, rp, vp, window, scale);
-    if (!latent_rows_mfma_supported(d) || (seq * heads + 15) / 16 > kMaxGridYZ || (batch * seq + 15) / 16 > kMaxGridYZ)
-        return fail(ASTRAI_MIX_UNSUPPORTED, "latent_rows: latent %lld + %lld (at most 1024, 1152 together) or too many rows",
+    if (!latent_rows_mfma_supported(d) || seq * heads * nsplit > kMaxInt || (batch * seq + 15) / 16 > kMaxGridYZ ||
+        batch * seq * heads > kMaxInt || max_len * (rp + dr) * 2 >= kMaxInt)
+        return fail(ASTRAI_MIX_UNSUPPORTED, "latent_rows: latent %lld + %lld (at most 1024, 64), too many rows or a sequence of 2 GiB",
                     (long long)rp, (long long)dr);
-    LatentRowsArgs a = {proj, ld, (int)g_off, w_ukv, w_uk_t, cache, positions, q_abs, nullptr, ws, out,
+    LatentRowsArgs a = {proj, ld, (int)g_off, w_ukv, cache, positions, q_abs, q_abs, ws, out,
                         (int)batch, (int)seq, (int)max_len, (int)nsplit};
     launch_latent_rows_mfma(a, d, static_cast<hipStream_t>(stream));
     return check_launch("latent_rows");
@@ -289,7 +300,7 @@ int astrai_mix_latent_rows_general(const void* proj, int64_t ld, int64_t g_off, 
     if (!latent_rows_general_supported(d))
         return fail(ASTRAI_MIX_UNSUPPORTED, "latent_rows_general: latent %lld, rotated %lld (at most 2048, 512)",
                     (long long)rp, (long long)dr);
-    LatentRowsArgs a = {proj, ld, (int)g_off, w_ukv, nullptr, cache, positions, nullptr, nullptr, nullptr, out,
+    LatentRowsArgs a = {proj, ld, (int)g_off, w_ukv, cache, positions, nullptr, nullptr, nullptr, out,
                         (int)batch, (int)seq, (int)max_len, 1};
     launch_latent_rows_general(a, d, dtype, static_cast<hipStream_t>(stream));
     return check_launch("latent_rows_general");

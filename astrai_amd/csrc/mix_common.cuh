@@ -11,6 +11,7 @@ namespace astrai_mix {
 
 using w8a8::block_sum;
 using w8a8::f32_to_bf16;
+using w8a8::f32x2;
 using w8a8::f32x4;
 using w8a8::kRowThreads;
 using w8a8::kWave;

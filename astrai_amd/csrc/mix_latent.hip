@@ -2,15 +2,17 @@
 // W_uk c, W_uv c of a cached latent c, plus one rotated key part shared by all heads.
 //
 //   latent_append   rotates the queries' rotated parts in place, norms the new latents, rotates
-//                   the new key parts and writes both into the cache
+//                   the new key parts and writes both into the cache; for the rows path it also absorbs
+//                   W_uk into the queries
 //   rows path       a few new tokens against the cache without ever forming keys or values:
 //                   q_u . (W_uk c) = (W_uk^T q_u) . c, and the output is W_uv (sum p c). With the
 //                   projection absorbed into the query, all heads of a token share one key/value
 //                   row per position, so the cache is read once per 16 (token, head) rows.
-//     absorb          q_abs[t, h] = W_uk[h]^T q_u[t, h]            (MFMA, weight-streaming)
-//     partial         split-context attention in the latent space  (MFMA)
-//     merge + expand  splits merged, W_uv[h] applied, output gate   (MFMA, weight-streaming)
-//   general path    the same three steps on the vector ALU for any size and for float
+//     absorb        q_abs[t, h] = W_uk[h]^T q_u[t, h]            (MFMA, weight-streaming)
+//     partial       split-context attention in the latent space  (MFMA)
+//     merge         splits of a row into one attended latent
+//     expand        W_uv[h] applied, output gate                 (MFMA, weight-streaming)
+//   general path  the same steps on the vector ALU for any size and for float, one kernel
 #include "mix_common.cuh"
 #include "mix_launchers.h"
 
@@ -18,19 +20,17 @@ namespace astrai_mix {
 
 namespace {
 
-// ---- append: one wave per token -----------------------------------------------------------------
-template <typename T>
-__global__ __launch_bounds__(256) void latent_append_kernel(LatentAppendArgs a, LatentDims d) {
-    const int lane = threadIdx.x & 63;
-    const int64_t t = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-    if (t >= a.tokens) return;
+// ---- append: N threads (a wave or a workgroup) per token --------------------------------------------
+template <typename T, int N>
+__device__ __forceinline__ void append_token(const LatentAppendArgs& a, const LatentDims& d, int64_t t, int lane,
+                                             float* slots) {
     const int64_t b = t / a.seq;
     const int64_t pos = a.positions[t - b * a.seq];
-    if (pos < 0 || pos >= a.max_len || pos >= a.rot_rows) return;
+    if (pos < 0 || pos >= a.max_len || pos >= a.rot_rows) return;   // (the same for the token's N threads)
     T* row = static_cast<T*>(a.proj) + t * a.ld;
     const float2* rot = reinterpret_cast<const float2*>(a.rot) + pos * a.half;
     const int qs = d.dn + d.dr;
-    for (int i = lane; i < d.heads * a.half; i += 64) {
+    for (int i = lane; i < d.heads * a.half; i += N) {
         const int h = i / a.half, p = i - h * a.half;
         T* u = row + h * qs + d.dn + p;
         const float2 cs = rot[p];
@@ -42,12 +42,12 @@ __global__ __launch_bounds__(256) void latent_append_kernel(LatentAppendArgs a, 
     const T* src = row + a.dkv_off;
     T* dst = static_cast<T*>(a.cache) + (b * a.max_len + pos) * (d.rp + d.dr);
     float s = 0.0f;
-    for (int c = lane * 4; c < d.rp; c += 256) {
+    for (int c = lane * 4; c < d.rp; c += 4 * N) {
         const f32x4 v = Elem<T>::get4(src + c);
         s += (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]);
     }
-    const float r = 1.0f / sqrtf(wave_sum(s) / (float)a.kv_rank + a.eps);
-    for (int c = lane * 4; c < d.rp; c += 256) {
+    const float r = 1.0f / sqrtf((N == 64 ? wave_sum(s) : block_sum(s, slots)) / (float)a.kv_rank + a.eps);
+    for (int c = lane * 4; c < d.rp; c += 4 * N) {
         f32x4 v = Elem<T>::get4(src + c);
         const f32x4 w = *reinterpret_cast<const f32x4*>(a.norm_w + c);
 #pragma unroll
@@ -56,63 +56,79 @@ __global__ __launch_bounds__(256) void latent_append_kernel(LatentAppendArgs a, 
     }
     src += d.rp;
     dst += d.rp;
-    for (int p = lane; p < a.half; p += 64) {
+    for (int p = lane; p < a.half; p += N) {
         const float2 cs = rot[p];
         const float x = Elem<T>::get(src + p), y = Elem<T>::get(src + p + a.half);
         Elem<T>::put(dst + p, x * cs.x - y * cs.y);
         Elem<T>::put(dst + p + a.half, y * cs.x + x * cs.y);
     }
-    for (int p = 2 * a.half + lane; p < d.dr; p += 64) dst[p] = src[p];
+    for (int p = 2 * a.half + lane; p < d.dr; p += N) dst[p] = src[p];
 }
 
-// ---- absorb (bf16): q_abs[t, h, r] = sum_d q[t, h, d] w_uk_t[h, r, d] ------------------------------
-// One workgroup per (64 latent columns, head, 16 tokens), a wave per 16 columns. Weight rows are the
-// MFMA's rows and tokens its columns, so a lane ends up with four consecutive latent columns of one
-// token. Both operands come straight from memory, 16 bytes a lane.
-__global__ __launch_bounds__(256) void latent_absorb_kernel(LatentRowsArgs a, LatentDims d) {
-    const int lane = threadIdx.x & 63, c16 = lane & 15, g = lane >> 4;
-    const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-    const int r0 = (int)blockIdx.x * 64 + wave * 16;
-    if (r0 >= d.rp) return;
-    const int h = blockIdx.y;
-    const int64_t tokens = (int64_t)a.batch * a.seq;
-    const int64_t t = (int64_t)blockIdx.z * 16 + c16;
-    const bool live = t < tokens;
-    const uint16_t* q = static_cast<const uint16_t*>(a.proj) + (live ? t : 0) * a.ld + h * (d.dn + d.dr) + 8 * g;
-    const uint16_t* w = static_cast<const uint16_t*>(a.w_uk_t) + ((int64_t)h * d.rp + r0 + c16) * d.dn + 8 * g;
-    f32x4 acc = {0, 0, 0, 0};
-    for (int k = 0; k < d.dn; k += 32) {
-        const u32x4 wf = *reinterpret_cast<const u32x4*>(w + k);
-        const u32x4 qf = live ? *reinterpret_cast<const u32x4*>(q + k) : u32x4{0, 0, 0, 0};
-        acc = mfma16(wf, qf, acc);
+// a wave per token (prompts)
+template <typename T>
+__global__ __launch_bounds__(256) void latent_append_kernel(LatentAppendArgs a, LatentDims d) {
+    const int64_t t = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (t < a.tokens) append_token<T, 64>(a, d, t, threadIdx.x & 63, nullptr);
+}
+
+// A few tokens: the first a.tokens workgroups append one each. The others absorb W_uk into the queries,
+//   q_abs[t, h, r] = sum_d q[t, h, d] w_uk_t[h, r, d]
+// over the unrotated columns, which the append leaves alone: one wave per (16 latent columns, head, 16
+// tokens). Weight rows are the MFMA's rows and tokens its columns, so a lane ends up with four consecutive
+// columns of one token; both operands come straight from memory, 16 bytes a lane.
+template <typename T>
+__global__ __launch_bounds__(256) void latent_append_few_kernel(LatentAppendArgs a, LatentDims d) {
+    __shared__ float slots[kRowThreads / kWave];
+    if ((int64_t)blockIdx.x < a.tokens) {
+        append_token<T, 256>(a, d, blockIdx.x, threadIdx.x, slots);
+        return;
     }
-    if (live)
-        Elem<uint16_t>::put4(static_cast<uint16_t*>(a.q_abs) + (t * d.heads + h) * d.rp + r0 + 4 * g, acc);
+    if constexpr (sizeof(T) == 2) {
+        const int nb = (d.rp + 63) / 64;
+        int item = (int)((int64_t)blockIdx.x - a.tokens);
+        const int lane = threadIdx.x & 63, c16 = lane & 15, g = lane >> 4;
+        const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+        const int r0 = ((item % nb) * 4 + wave) * 16;
+        item /= nb;
+        const int h = item % d.heads;
+        const int64_t t = (int64_t)(item / d.heads) * 16 + c16;
+        if (r0 >= d.rp) return;
+        const int64_t tl = min(t, a.tokens - 1);   // (a row past the end repeats the last one and is not stored)
+        const uint16_t* x = static_cast<const uint16_t*>(a.proj) + tl * a.ld + h * (d.dn + d.dr) + 8 * g;
+        const uint16_t* w = static_cast<const uint16_t*>(a.w_uk_t) + ((int64_t)h * d.rp + r0 + c16) * d.dn + 8 * g;
+        f32x4 acc = {0, 0, 0, 0};
+#pragma unroll 4
+        for (int k = 0; k < d.dn; k += 32)
+            acc = mfma16(*reinterpret_cast<const u32x4*>(w + k), *reinterpret_cast<const u32x4*>(x + k), acc);
+        if (t < a.tokens)
+            Elem<uint16_t>::put4(static_cast<uint16_t*>(a.q_abs) + (t * d.heads + h) * d.rp + r0 + 4 * g, acc);
+    }
 }
 
 // ---- split-context attention over the latent rows (bf16) -------------------------------------------
 // Rows are (token, head) pairs of one sequence, token-major; a workgroup takes 16 of them and one
 // split of the keys, in tiles of 32. Four waves:
-//   scores   wave (kh, ch) multiplies keys 16 kh .. of the tile with half ch of the row's 32-element
-//            steps; its key operand comes straight from the cache, and the same registers are
-//            written to LDS for the value product. The two halves meet in LDS.
+//   scores   wave (kh, ch) multiplies keys 16 kh .. of the tile with latent steps RH ch .. RH ch + RH - 1 (of
+//            32 columns) and rotated step ch; its key operand comes straight from the cache, and the
+//            latent registers are written to LDS for the value product. The halves meet in LDS.
 //   softmax  fp32, every wave for itself: lane (query c16, group g) holds keys 8g .. 8g+7, which is
 //            the value product's operand layout. Probabilities go in as two bf16 terms.
 //   values   wave w accumulates latent columns 16 (w + 4 i) .., the transposed operand out of LDS.
-// The LDS tiles alternate between two buffers: one barrier per tile.
-// KS: steps per half (compile time), also the bound on a wave's column tiles.
-template <int KS>
-__global__ __launch_bounds__(256) void latent_partial_kernel(LatentRowsArgs a, LatentDims d) {
+// The LDS tiles alternate between two buffers: one barrier per tile; key operands are requested two
+// tiles ahead. Nothing in a tile branches: with fewer latent columns than 64 RH, the steps past them
+// meet zero query operands and fill LDS columns that are never stored.
+template <int RH>
+__global__ __launch_bounds__(256, RH <= 8 ? 2 : 1) void latent_partial_kernel(LatentRowsArgs a, LatentDims d) {
     constexpr int kScRow = 36;                       // floats per query row of scores (32 + padding)
+    constexpr int kVRow = RH * 128 + 32;             // bytes per latent row in LDS
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
     const int lane = threadIdx.x & 63, c16 = lane & 15, g = lane >> 4;
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int kh = wave & 1, ch = wave >> 1;
-    const int split = blockIdx.x, rt = blockIdx.y, b = blockIdx.z;
+    const int split = (int)blockIdx.x % a.nsplit, rt = (int)blockIdx.x / a.nsplit, b = blockIdx.y;
     const int rows = a.seq * d.heads;
-    const int vrow = d.rp * 2 + 32;                  // bytes per latent row in LDS
-    uint8_t* vt = lds;
-    float* sc = reinterpret_cast<float*>(lds + 2 * 32 * vrow);
+    float* sc = reinterpret_cast<float*>(lds + 2 * 32 * kVRow);
 
     const int row = rt * 16 + c16;
     const bool live = row < rows;
@@ -127,69 +143,65 @@ __global__ __launch_bounds__(256) void latent_partial_kernel(LatentRowsArgs a, L
     const int tps = (tiles + a.nsplit - 1) / a.nsplit;
     const int t0 = split * tps, t1 = min(t0 + tps, tiles);
 
-    const int64_t ldc = d.rp + d.dr;
-    const int steps = (int)(ldc >> 5);
-    const int half_steps = (steps + 1) >> 1;
-    const int st0 = ch * half_steps, nst = min(half_steps, steps - st0);
-    // query operand of this wave's steps
-    u32x4 qf[KS];
+    const u32x4 zero = {0, 0, 0, 0};
+    u32x4 qf[RH + 1];   // query operand of this wave's steps; the rotated one last
     {
         const int64_t t = (int64_t)b * a.seq + tok;
         const uint16_t* qa = static_cast<const uint16_t*>(a.q_abs) + (t * d.heads + head) * d.rp;
-        const uint16_t* qr = static_cast<const uint16_t*>(a.proj) + t * a.ld + head * (d.dn + d.dr) + d.dn - d.rp;
+        const uint16_t* qr = static_cast<const uint16_t*>(a.proj) + t * a.ld + head * (d.dn + d.dr) + d.dn;
 #pragma unroll
-        for (int i = 0; i < KS; ++i) {
-            const int e = (st0 + i) * 32 + 8 * g;
-            qf[i] = (i < nst && live) ? *reinterpret_cast<const u32x4*>((e < d.rp ? qa : qr) + e) : u32x4{0, 0, 0, 0};
+        for (int i = 0; i < RH; ++i) {
+            const int e = (ch * RH + i) * 32 + 8 * g;
+            qf[i] = (e < d.rp && live) ? *reinterpret_cast<const u32x4*>(qa + e) : zero;
         }
+        qf[RH] = (ch * 32 < d.dr && live) ? *reinterpret_cast<const u32x4*>(qr + ch * 32 + 8 * g) : zero;
     }
-    const uint16_t* cache = static_cast<const uint16_t*>(a.cache) + (int64_t)b * a.max_len * ldc + st0 * 32 + 8 * g;
-    u32x4 kf[KS];
-    auto fetch = [&](int t) {
-        const int key = kmin + t * 32 + kh * 16 + c16;
-        const bool ok = t < t1 && key <= kmax;
-        const uint16_t* p = cache + (int64_t)(ok ? key : 0) * ldc;
+    // keys past kmax read as zeros
+    const uint32_t ldc = (uint32_t)(d.rp + d.dr) * 2;   // bytes
+    const __amdgpu_buffer_rsrc_t rc = w8a8::make_rsrc(
+        static_cast<const uint8_t*>(a.cache) + (int64_t)b * a.max_len * ldc, (uint32_t)(kmax + 1) * ldc);
+    const uint32_t lane_c = (uint32_t)(ch * RH * 64 + 16 * g), lane_r = (uint32_t)(d.rp * 2 + ch * 64 + 16 * g);
+    u32x4 ka[RH + 1], kb[RH + 1];   // key operands of two tiles in flight
+    auto fetch = [&](int t, u32x4 (&kf)[RH + 1]) {
+        const uint32_t off = t < t1 ? (uint32_t)(kmin + t * 32 + kh * 16 + c16) * ldc : w8a8::kOutOfRange;
 #pragma unroll
-        for (int i = 0; i < KS; ++i)
-            kf[i] = (ok && i < nst) ? *reinterpret_cast<const u32x4*>(p + i * 32) : u32x4{0, 0, 0, 0};
+        for (int i = 0; i < RH; ++i) kf[i] = w8a8::buf_load16(rc, off + lane_c + i * 64, 0);
+        kf[RH] = w8a8::buf_load16(rc, ch * 32 < d.dr ? off + lane_r : w8a8::kOutOfRange, 0);
     };
-    fetch(t0);
+    fetch(t0, ka);
+    fetch(t0 + 1, kb);
 
-    f32x4 acc[KS];
+    f32x4 acc[RH];
 #pragma unroll
-    for (int i = 0; i < KS; ++i) acc[i] = f32x4{0, 0, 0, 0};
-    float m = kNegBig, l = 0.0f;
+    for (int i = 0; i < RH; ++i) acc[i] = f32x4{0, 0, 0, 0};
+    float m = kNegBig, l = 0.0f;   // l: this lane's keys only
     const float c = d.scale * kLog2e;
-    const int rtiles = d.rp >> 4;
-    int buf = 0;
-    for (int t = t0; t < t1; ++t, buf ^= 1) {
-        uint8_t* v = vt + buf * 32 * vrow;
+    auto tile = [&](int t, int buf, u32x4 (&kf)[RH + 1]) {
+        uint8_t* v = lds + buf * 32 * kVRow;
         float* s = sc + buf * 2 * 16 * kScRow;
-        f32x4 part = {0, 0, 0, 0};
+        f32x4 part[2] = {{0, 0, 0, 0}, {0, 0, 0, 0}};
 #pragma unroll
-        for (int i = 0; i < KS; ++i) {
-            if (i < nst) {
-                part = mfma16(kf[i], qf[i], part);
-                const int e = (st0 + i) * 32 + 8 * g;
-                if (e < d.rp) *reinterpret_cast<u32x4*>(v + (kh * 16 + c16) * vrow + e * 2) = kf[i];
-            }
+        for (int i = 0; i <= RH; ++i) {
+            part[i & 1] = mfma16(kf[i], qf[i], part[i & 1]);
+            if (i < RH)
+                *reinterpret_cast<u32x4*>(v + (kh * 16 + c16) * kVRow + (ch * RH + i) * 64 + 16 * g) = kf[i];
         }
-        *reinterpret_cast<f32x4*>(s + (ch * 16 + c16) * kScRow + kh * 16 + 4 * g) = part;
-        fetch(t + 1);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) part[0][e] += part[1][e];
+        *reinterpret_cast<f32x4*>(s + (ch * 16 + c16) * kScRow + kh * 16 + 4 * g) = part[0];
+        fetch(t + 2, kf);
         __syncthreads();
         float p[8], tm = kNegBig;
-        {
-            const float* s0 = s + c16 * kScRow + 8 * g;
-            const float* s1 = s0 + 16 * kScRow;
+        const float* s0 = s + c16 * kScRow + 8 * g;
+        const float* s1 = s0 + 16 * kScRow;
 #pragma unroll
-            for (int e = 0; e < 8; e += 4) {
-                const f32x4 x = *reinterpret_cast<const f32x4*>(s0 + e), y = *reinterpret_cast<const f32x4*>(s1 + e);
+        for (int e = 0; e < 8; e += 4) {
+            const f32x4 x = *reinterpret_cast<const f32x4*>(s0 + e), y = *reinterpret_cast<const f32x4*>(s1 + e);
 #pragma unroll
-                for (int j = 0; j < 4; ++j) {
-                    const int key = kmin + t * 32 + 8 * g + e + j;
-                    p[e + j] = (key <= q_pos && key >= q_lo) ? (x[j] + y[j]) * c : kNegBig;
-                    tm = fmaxf(tm, p[e + j]);
-                }
+            for (int j = 0; j < 4; ++j) {
+                const int key = kmin + t * 32 + 8 * g + e + j;
+                p[e + j] = (key <= q_pos && key >= q_lo) ? (x[j] + y[j]) * c : kNegBig;
+                tm = fmaxf(tm, p[e + j]);
             }
         }
         tm = fmaxf(tm, __shfl_xor(tm, 16, kWave));
@@ -197,15 +209,12 @@ __global__ __launch_bounds__(256) void latent_partial_kernel(LatentRowsArgs a, L
         const float m_new = fmaxf(m, tm);
         const float alpha = __builtin_amdgcn_exp2f(m - m_new);
         m = m_new;
-        float ps = 0.0f;
+        l *= alpha;
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
             p[e] = p[e] > 0.5f * kNegBig ? __builtin_amdgcn_exp2f(p[e] - m_new) : 0.0f;
-            ps += p[e];
+            l += p[e];
         }
-        ps += __shfl_xor(ps, 16, kWave);
-        ps += __shfl_xor(ps, 32, kWave);
-        l = l * alpha + ps;
         u32x4 hi, lo;
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
@@ -215,28 +224,29 @@ __global__ __launch_bounds__(256) void latent_partial_kernel(LatentRowsArgs a, L
             lo[e] = l2;
         }
         // transposed latent operand: 16 columns x 32 keys, lane group g takes keys 8g .. 8g+7
-        const uint8_t* src = v + (8 * g + (c16 >> 2)) * vrow + (c16 & 3) * 8;
+        const uint8_t* src = v + (8 * g + (c16 >> 2)) * kVRow + (c16 & 3) * 8 + wave * 32;
 #pragma unroll
-        for (int i = 0; i < KS; ++i) {
-            const int rti = wave + 4 * i;
-            if (rti < rtiles) {
-                const uint8_t* q = src + rti * 32;
-                const u32x4 vf = join(lds_read_tr(q), lds_read_tr(q + 4 * vrow));
-                f32x4 o = acc[i];
+        for (int i = 0; i < RH; ++i) {
+            const u32x4 vf = join(lds_read_tr(src + i * 128), lds_read_tr(src + i * 128 + 4 * kVRow));
 #pragma unroll
-                for (int e = 0; e < 4; ++e) o[e] *= alpha;
-                o = mfma16(vf, hi, o);
-                acc[i] = mfma16(vf, lo, o);
-            }
+            for (int e = 0; e < 4; ++e) acc[i][e] *= alpha;
+            acc[i] = mfma16(vf, hi, acc[i]);
+            acc[i] = mfma16(vf, lo, acc[i]);
         }
+    };
+    for (int t = t0; t < t1; t += 2) {
+        tile(t, 0, ka);
+        if (t + 1 < t1) tile(t + 1, 1, kb);
     }
+    l += __shfl_xor(l, 16, kWave);
+    l += __shfl_xor(l, 32, kWave);
     if (!live) return;
     // workspace per (row, split): rp values, then maximum and sum
     float* w = a.ws + (((int64_t)b * rows + row) * a.nsplit + split) * (d.rp + 4);
 #pragma unroll
-    for (int i = 0; i < KS; ++i) {
-        const int rti = wave + 4 * i;
-        if (rti < rtiles) *reinterpret_cast<f32x4*>(w + rti * 16 + 4 * g) = acc[i];
+    for (int i = 0; i < RH; ++i) {
+        const int col = (wave + 4 * i) * 16;
+        if (col < d.rp) *reinterpret_cast<f32x4*>(w + col + 4 * g) = acc[i];
     }
     if (wave == 0 && g == 0) {
         w[d.rp] = m;
@@ -244,61 +254,58 @@ __global__ __launch_bounds__(256) void latent_partial_kernel(LatentRowsArgs a, L
     }
 }
 
-// ---- merge the splits, apply W_uv, gate (bf16) -------------------------------------------------------
-// One workgroup per (64 value columns, head, 16 tokens). Sixteen threads merge a token's splits
-// into LDS as bf16; then a wave per 16 value columns, as in absorb.
-constexpr int kMaxSplit = 64;
-
-__global__ __launch_bounds__(256) void latent_expand_kernel(LatentRowsArgs a, LatentDims d) {
-    extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
-    __shared__ float wt[16][kMaxSplit];
-    const int tid = threadIdx.x;
-    const int h = blockIdx.y;
-    const int64_t tokens = (int64_t)a.batch * a.seq;
-    const int orow = d.rp * 2 + 16;
-    {
-        const int i = tid >> 4, j = tid & 15;
-        const int64_t t = (int64_t)blockIdx.z * 16 + i;
-        const bool live = t < tokens;
-        const int64_t base = ((live ? t : 0) * d.heads + h) * a.nsplit;
-        const float* w = a.ws + base * (d.rp + 4);
-        float big = kNegBig, sum = 0.0f;
-        for (int s = 0; s < a.nsplit; ++s) big = fmaxf(big, w[(int64_t)s * (d.rp + 4) + d.rp]);
+// ---- merge the splits of a (token, head) row (bf16): one workgroup of 128 per row -------------------
+__global__ __launch_bounds__(128) void latent_merge_kernel(LatentRowsArgs a, LatentDims d) {
+    __shared__ float wt[kMaxSplit];
+    const int64_t row = blockIdx.x;
+    const int tid = threadIdx.x, lane = tid & 63;
+    const int ldw = d.rp + 4;
+    const float* w = a.ws + row * a.nsplit * ldw;
+    // (a split without a key has maximum kNegBig and sum 0)
+    const f32x2 ml = lane < a.nsplit ? *reinterpret_cast<const f32x2*>(w + (int64_t)lane * ldw + d.rp) : f32x2{kNegBig, 0.0f};
+    const float big = w8a8::wave_max(ml[0]);
+    const float e = __builtin_amdgcn_exp2f(ml[0] - big);
+    const float sum = wave_sum(ml[1] * e);
+    if (tid < a.nsplit) wt[tid] = sum > 0.0f ? e / sum : 0.0f;
+    __syncthreads();
+    for (int r = tid * 4; r < d.rp; r += 512) {
+        f32x4 o = {0, 0, 0, 0};
+#pragma unroll 4
         for (int s = 0; s < a.nsplit; ++s) {
-            const float* e = w + (int64_t)s * (d.rp + 4) + d.rp;
-            sum += e[1] * __builtin_amdgcn_exp2f(e[0] - big);
-        }
-        const float inv = (live && sum > 0.0f) ? 1.0f / sum : 0.0f;
-        for (int s = j; s < a.nsplit; s += 16)
-            wt[i][s] = __builtin_amdgcn_exp2f(w[(int64_t)s * (d.rp + 4) + d.rp] - big) * inv;
-        __syncthreads();
-        for (int r = j * 4; r < d.rp; r += 64) {
-            f32x4 o = {0, 0, 0, 0};
-            for (int s = 0; s < a.nsplit; ++s) {
-                const f32x4 v = *reinterpret_cast<const f32x4*>(w + (int64_t)s * (d.rp + 4) + r);
-                const float f = wt[i][s];
+            const f32x4 v = *reinterpret_cast<const f32x4*>(w + (int64_t)s * ldw + r);
+            const float f = wt[s];
 #pragma unroll
-                for (int e = 0; e < 4; ++e) o[e] += f * v[e];
-            }
-            Elem<uint16_t>::put4(reinterpret_cast<uint16_t*>(lds + i * orow) + r, o);
+            for (int j = 0; j < 4; ++j) o[j] += f * v[j];
         }
-        __syncthreads();
+        Elem<uint16_t>::put4(static_cast<uint16_t*>(a.o_lat) + row * d.rp + r, o);
     }
-    const int lane = tid & 63, c16 = lane & 15, g = lane >> 4;
-    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-    const int v0 = (int)blockIdx.x * 64 + wave * 16;
-    if (v0 >= d.vp) return;
-    const uint16_t* w = static_cast<const uint16_t*>(a.w_ukv) +
-                        ((int64_t)h * (d.dn + d.vp) + d.dn + v0 + c16) * d.rp + 8 * g;
-    const uint8_t* o = lds + c16 * orow + 16 * g;
-    f32x4 acc = {0, 0, 0, 0};
-    for (int k = 0; k < d.rp; k += 32)
-        acc = mfma16(*reinterpret_cast<const u32x4*>(w + k), *reinterpret_cast<const u32x4*>(o + k * 2), acc);
+}
+
+// ---- expand (bf16): out[t, h, v] = sigmoid(gate) sum_r o_lat[t, h, r] W_uv[h, v, r] --------------------
+// One workgroup per (16 value columns, head, 16 tokens), the waves sharing out the latent columns, so
+// that a wave's operands are one round of loads. Layouts as in absorb.
+__global__ __launch_bounds__(256) void latent_expand_kernel(LatentRowsArgs a, LatentDims d) {
+    __shared__ f32x4 part[3][64];
+    const int lane = threadIdx.x & 63, c16 = lane & 15, g = lane >> 4;
+    const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int v0 = (int)blockIdx.x * 16, h = blockIdx.y;
+    const int64_t tokens = (int64_t)a.batch * a.seq;
     const int64_t t = (int64_t)blockIdx.z * 16 + c16;
-    if (t >= tokens) return;
-    const float gate = sigmoid(Elem<uint16_t>::get(static_cast<const uint16_t*>(a.proj) + t * a.ld + a.g_off + h));
+    const int64_t tl = min(t, tokens - 1);
+    const float z = Elem<uint16_t>::get(static_cast<const uint16_t*>(a.proj) + tl * a.ld + a.g_off + h);
+    const uint16_t* x = static_cast<const uint16_t*>(a.o_lat) + (tl * d.heads + h) * d.rp + 8 * g;
+    const uint16_t* w = static_cast<const uint16_t*>(a.w_ukv) + ((int64_t)h * (d.dn + d.vp) + d.dn + v0 + c16) * d.rp + 8 * g;
+    f32x4 acc = {0, 0, 0, 0};
+#pragma unroll 4
+    for (int k = wave * 32; k < d.rp; k += 128)
+        acc = mfma16(*reinterpret_cast<const u32x4*>(w + k), *reinterpret_cast<const u32x4*>(x + k), acc);
+    if (wave) part[wave - 1][lane] = acc;
+    __syncthreads();
+    if (wave || t >= tokens) return;
+    const float gate = sigmoid(z);
 #pragma unroll
-    for (int e = 0; e < 4; ++e) acc[e] *= gate;
+    for (int e = 0; e < 4; ++e)
+        acc[e] = ((acc[e] + part[0][lane][e]) + (part[1][lane][e] + part[2][lane][e])) * gate;
     Elem<uint16_t>::put4(static_cast<uint16_t*>(a.out) + (t * d.heads + h) * d.vp + v0 + 4 * g, acc);
 }
 
@@ -386,43 +393,50 @@ __global__ __launch_bounds__(256) void latent_general_kernel(LatentRowsArgs a, L
     }
 }
 
-template <int KS>
+template <int RH>
 void partial_t(const LatentRowsArgs& a, const LatentDims& d, hipStream_t stream) {
-    const int rows = a.seq * d.heads;
-    const size_t shared = 2 * 32 * (size_t)(d.rp * 2 + 32) + 2 * 2 * 16 * 36 * sizeof(float);
-    static const hipError_t once = hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_partial_kernel<KS>),
-                                                       hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+    constexpr int shared = 2 * 32 * (RH * 128 + 32) + 2 * 2 * 16 * 36 * (int)sizeof(float);
+    static const hipError_t once = hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_partial_kernel<RH>),
+                                                       hipFuncAttributeMaxDynamicSharedMemorySize, shared);
     (void)once;
-    const dim3 grid((unsigned)a.nsplit, (unsigned)((rows + 15) / 16), (unsigned)a.batch);
-    latent_partial_kernel<KS><<<grid, 256, shared, stream>>>(a, d);
+    const int rows = a.seq * d.heads;
+    const dim3 grid((unsigned)a.nsplit * (unsigned)((rows + 15) / 16), (unsigned)a.batch);
+    latent_partial_kernel<RH><<<grid, 256, shared, stream>>>(a, d);
 }
 
 }  // namespace
 
 void launch_latent_append(const LatentAppendArgs& a, const LatentDims& d, int dtype, hipStream_t stream) {
-    const dim3 grid((unsigned)((a.tokens + 3) / 4));
-    if (dtype) latent_append_kernel<float><<<grid, 256, 0, stream>>>(a, d);
-    else latent_append_kernel<uint16_t><<<grid, 256, 0, stream>>>(a, d);
+    if (a.q_abs || a.tokens <= 1024) {
+        const int64_t absorb = a.q_abs ? (int64_t)((d.rp + 63) / 64) * d.heads * ((a.tokens + 15) / 16) : 0;
+        const dim3 grid((unsigned)(a.tokens + absorb));
+        if (dtype) latent_append_few_kernel<float><<<grid, 256, 0, stream>>>(a, d);
+        else latent_append_few_kernel<uint16_t><<<grid, 256, 0, stream>>>(a, d);
+    } else {
+        const dim3 grid((unsigned)((a.tokens + 3) / 4));
+        if (dtype) latent_append_kernel<float><<<grid, 256, 0, stream>>>(a, d);
+        else latent_append_kernel<uint16_t><<<grid, 256, 0, stream>>>(a, d);
+    }
 }
 
 // 1024 latent columns: two 32-row tiles of them are 130 KiB of LDS, the scores 9 KiB
-bool latent_rows_mfma_supported(const LatentDims& d) { return d.rp <= 1024 && d.rp + d.dr <= 1152; }
+bool latent_rows_mfma_supported(const LatentDims& d) { return d.rp <= 1024 && d.dr <= 64; }
 
 int64_t latent_rows_workspace_floats(const LatentDims& d, int64_t tokens, int nsplit) {
     return tokens * d.heads * nsplit * (d.rp + 4);
 }
 
 void launch_latent_rows_mfma(const LatentRowsArgs& a, const LatentDims& d, hipStream_t stream) {
-    const unsigned tt = (unsigned)(((int64_t)a.batch * a.seq + 15) / 16);
-    latent_absorb_kernel<<<dim3((unsigned)((d.rp + 63) / 64), (unsigned)d.heads, tt), 256, 0, stream>>>(a, d);
-    const int half = ((d.rp + d.dr) / 32 + 1) / 2;
-    if (half <= 2) partial_t<2>(a, d, stream);
-    else if (half <= 4) partial_t<4>(a, d, stream);
-    else if (half <= 6) partial_t<6>(a, d, stream);
-    else if (half <= 10) partial_t<10>(a, d, stream);
-    else partial_t<18>(a, d, stream);
-    const size_t shared = 16 * (size_t)(d.rp * 2 + 16);
-    latent_expand_kernel<<<dim3((unsigned)((d.vp + 63) / 64), (unsigned)d.heads, tt), 256, shared, stream>>>(a, d);
+    const int64_t tokens = (int64_t)a.batch * a.seq;
+    if (d.rp <= 64) partial_t<1>(a, d, stream);
+    else if (d.rp <= 128) partial_t<2>(a, d, stream);
+    else if (d.rp <= 256) partial_t<4>(a, d, stream);
+    else if (d.rp <= 384) partial_t<6>(a, d, stream);
+    else if (d.rp <= 512) partial_t<8>(a, d, stream);
+    else partial_t<16>(a, d, stream);
+    latent_merge_kernel<<<(unsigned)(tokens * d.heads), 128, 0, stream>>>(a, d);
+    latent_expand_kernel<<<dim3((unsigned)(d.vp / 16), (unsigned)d.heads, (unsigned)((tokens + 15) / 16)), 256, 0,
+                           stream>>>(a, d);
 }
 
 bool latent_rows_general_supported(const LatentDims& d) { return d.rp <= kGenRank && d.dr <= kGenDims; }

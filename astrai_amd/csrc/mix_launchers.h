@@ -44,6 +44,8 @@ struct LatentAppendArgs {
     const int64_t* positions;  // [seq]
     const float* norm_w;       // [rp]
     void* cache;               // [batch, max_len, rp + dr]
+    const void* w_uk_t;        // [heads, rp, dn], with q_abs (bf16)
+    void* q_abs;               // [batch * seq, heads, rp] or null
     int64_t tokens;            // batch * seq
     int64_t rot_rows;          // rows of `rot`
     int seq, max_len, half, kv_rank;
@@ -67,17 +69,17 @@ struct LatentPrefillArgs {
 bool latent_prefill_supported(const LatentDims& d);
 bool launch_latent_prefill(const LatentPrefillArgs& a, const LatentDims& d, hipStream_t stream);
 
+constexpr int kMaxSplit = 64;
 struct LatentRowsArgs {
     const void* proj;          // as above, q rotated
     int64_t ld;
     int g_off;
     const void* w_ukv;         // [heads * (dn + vp), rp]
-    const void* w_uk_t;        // [heads, rp, dn] (bf16 MFMA path only)
     const void* cache;
     const int64_t* positions;  // [seq]
-    void* q_abs;               // scratch [batch * seq, heads, rp]
-    void* o_lat;               // scratch [batch * seq, heads, rp] (general path)
-    float* ws;                 // scratch, latent_rows_workspace_floats (MFMA path)
+    const void* q_abs;         // [batch * seq, heads, rp] (MFMA path, as the next two)
+    void* o_lat;               // scratch [batch * seq, heads, rp], may be q_abs
+    float* ws;                 // scratch, latent_rows_workspace_floats
     void* out;                 // [batch, seq, heads * vp]
     int batch, seq, max_len, nsplit;
 };

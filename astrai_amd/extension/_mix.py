@@ -38,11 +38,11 @@ PROTOTYPES = {
     "astrai_mix_silu_mul": ([_P, _P, _I64, _I64, _INT, _P], _INT),
     "astrai_mix_gated_rms_norm": ([_P, _P, _I64, _P, _P, _I64, _I64, _I64, _F32, _INT, _P], _INT),
     "astrai_mix_latent_append": (
-        [_P, _I64, _I64, _P, _I64, _I64, _P, _P, _P] + [_I64] * 8 + [_F32, _INT, _P], _INT),
+        [_P, _I64, _I64, _P, _I64, _I64] + [_P] * 5 + [_I64] * 8 + [_F32, _INT, _P], _INT),
     "astrai_mix_latent_prefill": ([_P, _I64, _I64, _P, _P, _P] + [_I64] * 12 + [_F32, _P], _INT),
     "astrai_mix_latent_rows_workspace_floats": ([_I64] * 4, _I64),
     "astrai_mix_latent_rows": (
-        [_P, _I64, _I64, _P, _P, _P, _P, _P, _P, _P] + [_I64] * 9 + [_F32, _I64, _P], _INT),
+        [_P, _I64, _I64] + [_P] * 6 + [_I64] * 9 + [_F32, _I64, _P], _INT),
     "astrai_mix_latent_rows_general": ([_P, _I64, _I64, _P, _P, _P, _P] + [_I64] * 9 + [_F32, _INT, _P], _INT),
     "astrai_mix_lightning_chunk": ([_P] + [_I64] * 4 + [_P] * 4 + [_I64] * 6 + [_P], _INT),
     "astrai_mix_lightning_step": ([_P] + [_I64] * 4 + [_P] * 3 + [_I64] * 5 + [_INT, _P], _INT),
@@ -244,9 +244,11 @@ def _latent_block(what: str, s: LatentShape, proj, cache, positions):
 
 
 def latent_append(proj: torch.Tensor, s: LatentShape, dkv_off: int, rot: torch.Tensor, positions: torch.Tensor,
-                  norm_w: Optional[torch.Tensor], cache: torch.Tensor, eps: float) -> None:
+                  norm_w: Optional[torch.Tensor], cache: torch.Tensor, eps: float,
+                  w_uk_t: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
     """Rotate the queries of ``proj [batch * seq, ld]`` in place and, with ``dkv_off >= 0``, write the
-    normed latents and rotated key parts into ``cache [batch, max_len, rp + dr]`` at ``positions``."""
+    normed latents and rotated key parts into ``cache [batch, max_len, rp + dr]`` at ``positions``. With
+    ``w_uk_t [heads, rp, dn]`` (bf16) the absorbed queries ``[batch * seq, heads, rp]`` are returned."""
     lib = _require()
     batch, seq, max_len = _latent_block("latent_append", s, proj, cache, positions)
     _dense("latent_append", torch.float32, rot)
@@ -255,15 +257,25 @@ def latent_append(proj: torch.Tensor, s: LatentShape, dkv_off: int, rot: torch.T
     if dkv_off >= 0:
         _dense("latent_append", torch.float32, norm_w)
         _shape("latent_append", norm_w, s.rp)
+    q_abs = None
+    if w_uk_t is not None:
+        _dense("latent_append", torch.bfloat16, proj, w_uk_t)
+        _shape("latent_append", w_uk_t, s.heads, s.rp, s.dn)
     with _on_device(proj.device):
+        if w_uk_t is not None:
+            q_abs = torch.empty((proj.size(0), s.heads, s.rp), device=proj.device, dtype=proj.dtype)
         _check(lib.astrai_mix_latent_append(
             proj.data_ptr(), proj.size(1), dkv_off, rot.data_ptr(), rot.size(0), rot.size(1), positions.data_ptr(),
-            norm_w.data_ptr() if dkv_off >= 0 else None, cache.data_ptr(), batch, seq, max_len, s.heads, s.dn, s.dr,
+            norm_w.data_ptr() if dkv_off >= 0 else None, cache.data_ptr(), None if w_uk_t is None else w_uk_t.data_ptr(),
+            None if q_abs is None else q_abs.data_ptr(), batch, seq, max_len, s.heads, s.dn, s.dr,
             s.rp, s.kv_rank, eps, _dtype(proj, "latent_append"), _stream(proj)), lib)
+    return q_abs
 
 
 def latent_prefill_supported(s: LatentShape) -> bool:
-    return s.dn + s.dr <= 256 and s.vp <= 128
+    """Sizes the matrix-core prompt kernel takes (the limits its entry point checks)."""
+    return (s.dn <= 128 and s.dr <= 64 and s.vp <= 128 and 1e-4 <= s.scale <= 1e4
+            and 128 * s.heads * (s.dn + s.vp) < 1 << 30)
 
 
 def latent_prefill(proj: torch.Tensor, s: LatentShape, g_off: int, kv: torch.Tensor, cache: torch.Tensor,
@@ -284,8 +296,9 @@ def latent_prefill(proj: torch.Tensor, s: LatentShape, g_off: int, kv: torch.Ten
     return out
 
 
-def latent_rows_supported(s: LatentShape) -> bool:
-    return s.rp <= 1024 and s.rp + s.dr <= 1152
+def latent_rows_supported(s: LatentShape, max_len: int) -> bool:
+    """Sizes the matrix-core kernels of :func:`latent_rows` take (the limits its entry point checks)."""
+    return s.rp <= 1024 and s.dr <= 64 and max_len * s.cache_cols * 2 < 0x7fffffff
 
 
 def latent_rows_nsplit(s: LatentShape, batch: int, seq: int, max_len: int) -> int:
@@ -296,11 +309,12 @@ def latent_rows_nsplit(s: LatentShape, batch: int, seq: int, max_len: int) -> in
     return max(1, min(-(-512 // groups), tiles // 4, MAX_SPLIT))
 
 
-def latent_rows(proj: torch.Tensor, s: LatentShape, g_off: int, w_ukv: torch.Tensor, w_uk_t: Optional[torch.Tensor],
-                cache: torch.Tensor, positions: torch.Tensor) -> torch.Tensor:
+def latent_rows(proj: torch.Tensor, s: LatentShape, g_off: int, w_ukv: torch.Tensor, cache: torch.Tensor,
+                positions: torch.Tensor, q_abs: Optional[torch.Tensor] = None, nsplit: int = 0) -> torch.Tensor:
     """The same attention computed in the latent space, for a few new tokens (positions on the
-    device). ``w_ukv [heads * (dn + vp), rp]``, ``w_uk_t [heads, rp, dn]``. bf16 within the matrix-core
-    kernels' sizes runs on those, everything else on the general kernel."""
+    device). ``w_ukv [heads * (dn + vp), rp]``. With the absorbed queries ``q_abs`` of
+    :func:`latent_append` (overwritten here) on the matrix cores, ``nsplit`` 0 picking a split count;
+    without them on the general kernel, bf16 or float."""
     lib = _require()
     batch, seq, max_len = _latent_block("latent_rows", s, proj, cache, positions)
     _dense("latent_rows", proj.dtype, proj, w_ukv)
@@ -308,17 +322,16 @@ def latent_rows(proj: torch.Tensor, s: LatentShape, g_off: int, w_ukv: torch.Ten
     n, dev = proj.size(0), proj.device
     with _on_device(dev):
         out = torch.empty((n, s.heads * s.vp), device=dev, dtype=proj.dtype)
-        if proj.dtype == torch.bfloat16 and latent_rows_supported(s):
-            _dense("latent_rows", proj.dtype, w_uk_t)
-            _shape("latent_rows", w_uk_t, s.heads, s.rp, s.dn)
-            nsplit = latent_rows_nsplit(s, batch, seq, max_len)
-            q_abs = torch.empty((n, s.heads, s.rp), device=dev, dtype=proj.dtype)
+        if q_abs is not None:
+            _dense("latent_rows", torch.bfloat16, proj, q_abs)
+            _shape("latent_rows", q_abs, n, s.heads, s.rp)
+            nsplit = nsplit or latent_rows_nsplit(s, batch, seq, max_len)
             ws = torch.empty(lib.astrai_mix_latent_rows_workspace_floats(n, s.heads, s.rp, nsplit), device=dev,
                              dtype=torch.float32)
             _check(lib.astrai_mix_latent_rows(
-                proj.data_ptr(), proj.size(1), g_off, w_ukv.data_ptr(), w_uk_t.data_ptr(), cache.data_ptr(),
-                positions.data_ptr(), q_abs.data_ptr(), ws.data_ptr(), out.data_ptr(), batch, seq, max_len, s.heads,
-                s.dn, s.dr, s.rp, s.vp, s.window, s.scale, nsplit, _stream(proj)), lib)
+                proj.data_ptr(), proj.size(1), g_off, w_ukv.data_ptr(), cache.data_ptr(), positions.data_ptr(),
+                q_abs.data_ptr(), ws.data_ptr(), out.data_ptr(), batch, seq, max_len, s.heads, s.dn, s.dr, s.rp, s.vp,
+                s.window, s.scale, nsplit, _stream(proj)), lib)
         else:
             _check(lib.astrai_mix_latent_rows_general(
                 proj.data_ptr(), proj.size(1), g_off, w_ukv.data_ptr(), cache.data_ptr(), positions.data_ptr(),

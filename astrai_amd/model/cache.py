@@ -59,9 +59,9 @@ class MixerCache(StepCache):
     def add_state(self, layer: int, *shape: int) -> None:
         self.state[layer] = torch.zeros((self.batch, *shape), device=self.device, dtype=torch.float32)
 
-    def add_rotary(self, key, build: Callable[[int], Tensor]) -> None:
+    def add_rotary(self, key, build: Callable[..., Tensor]) -> None:
         if key not in self.rotary:
-            self.rotary[key] = build(self.max_len).to(self.device)
+            self.rotary[key] = build(self.max_len, self.device)
 
     def reset(self) -> None:
         super().reset()

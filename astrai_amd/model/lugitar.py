@@ -56,6 +56,7 @@ def _latent_attention(cfg: LugitarConfig, i: int) -> LatentAttention:
         src = cfg.layers[source]["mixer"]
         if src.get("kv_from") is not None:
             raise ValueError(f"layer {i}: kv_from {source} has no latents of its own")
+        m = {**{key: src[key] for key in ("kv_rank", "rot_dim", "rot")}, **m}
         for key in ("kv_rank", "rot_dim", "rot"):
             if src[key] != m[key]:
                 raise ValueError(f"layer {i}: {key} differs from layer {source}, whose latents it reads")

@@ -160,14 +160,14 @@ class Rotation:
         yarn = None if s is None else (float(s["factor"]), float(s["original"]), float(s["fast"]), float(s["slow"]))
         return Rotation(int(d["dims"]), float(d["base"]), yarn)
 
-    def table(self, max_len: int) -> Tensor:
-        """``[max_len, dims / 2, 2]`` fp32 (cos, sin), YaRN's magnitude included."""
+    def table(self, max_len: int, device="cpu") -> Tensor:
+        """``[max_len, dims / 2, 2]`` fp32 (cos, sin) on ``device``, YaRN's magnitude included."""
         if self.yarn is None:
             freqs = self.base ** (-torch.arange(0, self.dims, 2, dtype=torch.float64) / self.dims)
-            return rotary_table(freqs, max_len)
+            return rotary_table(freqs.to(device), max_len)
         factor, original, fast, slow = self.yarn
-        return rotary_table(yarn_frequencies(self.dims, self.base, factor, original, fast, slow), max_len,
-                            0.1 * math.log(factor) + 1.0)
+        freqs = yarn_frequencies(self.dims, self.base, factor, original, fast, slow)
+        return rotary_table(freqs.to(device), max_len, 0.1 * math.log(factor) + 1.0)
 
 
 class LatentAttention(nn.Module):
@@ -227,14 +227,19 @@ class LatentAttention(nn.Module):
         latent = cache.latent[self.kv_layer]
         proj = self.in_proj(h)
         g_off = self.in_proj.offset["g"]
-        _mix.latent_append(proj, s, self.in_proj.offset.get("dkv", -1), cache.rotary[self.rotation], ctx.positions,
-                           self.latent_norm.weight if self.owns_latent else None, latent, self.eps)
-        if ctx.seq <= LATENT_ROWS_MAX or proj.dtype != torch.bfloat16 or not _mix.latent_prefill_supported(s):
-            out = _mix.latent_rows(proj, s, g_off, self.w_ukv, self.w_uk_t, latent, ctx.positions)
+        rows = ctx.seq <= LATENT_ROWS_MAX or proj.dtype != torch.bfloat16 or not _mix.latent_prefill_supported(s)
+        absorb = rows and self.w_uk_t is not None and _mix.latent_rows_supported(s, cache.max_len)
+        q_abs = _mix.latent_append(proj, s, self.in_proj.offset.get("dkv", -1), cache.rotary[self.rotation],
+                                   ctx.positions, self.latent_norm.weight if self.owns_latent else None, latent,
+                                   self.eps, self.w_uk_t if absorb else None)
+        if rows:
+            out = _mix.latent_rows(proj, s, g_off, self.w_ukv, latent, ctx.positions, q_abs)
         else:
             first = max(ctx.start - s.window + 1, 0)
             c = latent[:, first:ctx.start + ctx.seq, :s.rp]
-            kv = F.linear(c, self.w_ukv)
+            # (a plain 2-D product: a strided 3-D operand would go to a batched one)
+            kv = F.linear(c[0] if ctx.batch == 1 else c.reshape(-1, s.rp), self.w_ukv)
+            kv = kv.reshape(ctx.batch, -1, kv.size(-1))
             out = _mix.latent_prefill(proj, s, g_off, kv, latent, ctx.start, first)
         return self.o(out)
 

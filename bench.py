@@ -238,6 +238,180 @@ def _bench_decoder(dev):
     return res
 
 
+PEAK_BF16_TFLOPS = 2500.0  # MI355X dense bf16 MFMA
+
+
+def _lugitar_config(width, heads, ff, layers, window=1024, vocab=32000):
+    """A Lugitar model with layers of a real model's sizes: groups of four layers (latent attention,
+    lightning, latent attention on the first one's latents, lightning), latent 512 + 64, heads of 128."""
+    rot = {"dims": 64, "base": 10000.0, "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}
+    out = []
+    for i in range(layers):
+        if i % 2 == 0:
+            mixer = {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "rot": rot,
+                     "scale": 192 ** -0.5, "mask": {"size": window}}
+            if i % 4 == 2:
+                mixer["kv_from"] = i - 2
+            out.append({"type": "latent_attention", "mixer": mixer, "mlp": {"kind": "dense", "ff": ff}})
+        else:
+            decay = [1.0 - 2.0 ** (-2 - 6 * h / heads) for h in range(heads)]
+            out.append({"type": "lightning", "mixer": {"heads": heads, "dim": 128, "vdim": 128, "decay": decay},
+                        "mlp": {"kind": "dense", "ff": ff}})
+    return {"architecture": "Lugitar", "vocab": vocab, "width": width, "layers": out, "norm": {"eps": 1e-6},
+            "residual_mult": 0.5}
+
+
+def _lugitar_kernels(dev, width, heads, ff, batch, seq, window=1024):
+    """Every kernel of a Lugitar layer beside the like kernel of the dense decoder at equal size (heads of
+    128, 4 query heads per KV head), each as (microseconds, fraction of its roofline: the larger of bytes
+    over 8 TB/s and MFMA flops over 2.5 PFLOP/s bf16, over the time). Launches replayed as HIP graphs; each
+    pair's two sides are timed one after the other."""
+    import torch
+
+    from astrai_amd.extension import _cabi, _mix
+
+    bf, f32 = torch.bfloat16, torch.float32
+    n, hkv, d = batch * seq, heads // 4, 128
+    ctx = window                           # decode context, of both
+    shape = _mix.LatentShape(heads, d, 64, 512, d, 512, window, 192 ** -0.5)
+    cols, gc = shape.q_cols + shape.cache_cols + heads, heads
+    res = {}
+
+    def r(*size, dtype=bf, scale=1.0):
+        return (torch.randn(*size, device=dev) * scale).to(dtype)
+
+    def entry(name, fn, nbytes, flops=0.0, launches=20):
+        us = _graph_us(lambda i: fn(), launches)
+        roof = max(nbytes / (PEAK_HBM_GBS * 1e9), flops / (PEAK_BF16_TFLOPS * 1e12)) * 1e6
+        res[name] = {"us": round(us, 2), "roofline": round(roof / us, 3)}
+
+    # pairs a causal / windowed block of seq queries forms per head
+    causal = seq * (seq + 1) / 2
+    seen = sum(min(i + 1, window) for i in range(seq))
+    pos, last = torch.arange(seq, device=dev), torch.tensor([ctx - 1], device=dev)
+    # --- prompt attention
+    q, kc, vc = r(batch, heads, seq, d), r(batch, hkv, max(ctx, seq), d), r(batch, hkv, max(ctx, seq), d)
+    entry("dense attn_prefill", lambda: _cabi.attn_prefill(q, kc, vc, pos),
+          (2 * n * heads * d + 2 * n * hkv * d) * 2, 4 * d * heads * batch * causal)
+    proj, cache, kv = r(n, cols), r(batch, max(ctx, seq), 576), r(batch, seq, heads * 256)
+    entry("latent_prefill", lambda: _mix.latent_prefill(proj, shape, cols - gc, kv, cache, 0, 0),
+          (n * heads * (192 + 256 + d) + n * 64) * 2, 2 * (192 + d) * heads * batch * seen)
+    lproj, state = r(n, 4 * heads * d), torch.zeros(batch, heads, d, d, device=dev)
+    dec = _mix.decay_powers([0.5 + 0.49 * h / heads for h in range(heads)]).to(dev)
+    hd = heads * d
+    # chunked form, 64 tokens: scores, score x value (half of them hidden), state read, state update
+    entry("lightning chunk", lambda: _mix.lightning(lproj, 0, hd, 2 * hd, dec, state, False),
+          4 * n * hd * 2 + 2 * state.numel() * 4, n * heads * 2 * (32 * d + 32 * d + 2 * d * d))
+    # --- decode attention
+    q1, kc1, vc1 = r(batch, heads, 1, d), r(batch, hkv, ctx, d), r(batch, hkv, ctx, d)
+    entry("dense attn_decode", lambda: _cabi.attn_decode(q1, kc1, vc1, last), 2 * batch * hkv * ctx * d * 2)
+    p1, wukv, wukt = r(batch, cols), r(heads * 256, 512), r(heads, 512, d)
+    keys = min(ctx, window)
+    q_abs = r(batch, heads, 512)
+    entry("latent_rows", lambda: _mix.latent_rows(p1, shape, cols - gc, wukv, cache, last, q_abs),
+          batch * keys * 576 * 2 + wukv.numel(), 2 * batch * heads * (keys * (576 + 512) + 512 * d))
+    l1 = r(batch, 4 * hd)
+    entry("lightning step", lambda: _mix.lightning(l1, 0, hd, 2 * hd, dec, state, True), 2 * state.numel() * 4)
+    # --- row operations, prompt and decode
+    for tag, rows in (("prefill", n), ("decode", batch)):
+        x, y, w = r(rows, width), r(rows, width), torch.ones(width, device=dev, dtype=bf)
+        entry(f"dense add_rmsnorm_quantize {tag}", lambda: _cabi.add_rmsnorm_quantize_int8(x, w, 1e-5, y),
+              rows * width * (2 + 2 + 2 + 1))
+        xf, w32 = r(rows, width, dtype=f32), torch.ones(width, device=dev)
+        entry(f"residual_norm {tag}", lambda: _mix.residual_norm(y, xf, w32, w32, 0.5, 1e-6),
+              rows * width * (2 + 4 + 4 + 2))
+        gu = r(rows, 2 * ff)
+        entry(f"dense silu_mul_quantize {tag}", lambda: _cabi.silu_mul_quantize_int8(gu[:, :ff], gu[:, ff:]),
+              rows * ff * (4 + 1))
+        entry(f"silu_mul {tag}", lambda: _mix.silu_mul(gu), rows * ff * 6)
+        o, lp, wv = r(rows, hd), r(rows, 4 * hd), torch.ones(hd, device=dev)
+        entry(f"gated_rms_norm {tag}", lambda: _mix.gated_rms_norm(o, lp, 3 * hd, wv, hd, 1e-6), rows * hd * 6)
+        s1 = rows // batch
+        qkv, fr = r(batch, s1, (heads + 2 * hkv) * d), r(s1, d // 2, 2, dtype=f32)
+        ps = torch.arange(s1, device=dev)
+        entry(f"dense rope_cache_write {tag}", lambda: _cabi.rope_cache_write(qkv, fr, ps, kc, vc, heads, hkv, d),
+              2 * qkv.numel() * 2)
+        pj, rot, w5 = r(rows, cols), r(max(ctx, seq), 32, 2, dtype=f32), torch.ones(512, device=dev)
+        absorb = tag == "decode"
+        entry(f"latent_append {tag}" + " (+ absorbed queries)" * absorb,
+              lambda: _mix.latent_append(pj, shape, shape.q_cols, rot, ps, w5, cache, 1e-6, wukt if absorb else None),
+              rows * (2 * heads * 64 + 2 * 576) * 2 + absorb * (wukt.numel() + rows * heads * (d + 512)) * 2)
+    return res
+
+
+def _bench_lugitar(dev):
+    """Lugitar models (random weights, bf16) beside the dense GQA decoder of equal width, depth and feed-forward,
+    in its own bf16 form and in its fused int8 form: prompt and decode throughput, then the kernels."""
+    import torch
+
+    from astrai_amd.extension import w8a8
+    from astrai_amd.model import (AutoRegressiveLM, AutoRegressiveLMConfig, LugitarConfig, LugitarLM,
+                                  fuse_int8_weights, greedy_generate)
+
+    def timed(fn, reps=3):
+        for _ in range(2):
+            fn()
+        ts = []
+        for _ in range(reps):
+            torch.cuda.synchronize()
+            t0 = time.perf_counter()
+            fn()
+            torch.cuda.synchronize()
+            ts.append(time.perf_counter() - t0)
+        return sorted(ts)[len(ts) // 2]
+
+    out = {"models": [], "kernels": []}
+    cases = [(2048, 16, 5632, 24, 32, 512, 64), (2048, 16, 5632, 24, 1, 4096, 64), (4096, 32, 8192, 8, 8, 2048, 64)]
+    for width, heads, ff, layers, batch, prompt, steps in cases:
+        row = {"width": width, "layers": layers, "ff": ff, "heads": heads, "batch": batch, "prompt": prompt}
+        ids = torch.randint(0, 32000, (batch, prompt), generator=torch.Generator().manual_seed(4)).to(dev)
+
+        def legs(tag, model):
+            with torch.no_grad():
+                last = torch.tensor([prompt - 1], device=dev)
+
+                def prefill():
+                    return model(ids, model.new_cache(batch, prompt + steps), logits_at=last)["logits"]
+
+                t_pre = timed(prefill)
+                t_all = timed(lambda: greedy_generate(model, ids, steps, use_graph=True))
+                # (greedy_generate forms the whole prompt's logits: its own prefill is timed with them)
+                t_gen0 = timed(lambda: greedy_generate(model, ids, 1, use_graph=True))
+                # two eager steps and the capture are in t_all: a second, longer run takes them out
+                t_long = timed(lambda: greedy_generate(model, ids, 2 * steps, use_graph=True))
+                step = (t_long - t_all) / steps
+                row[tag] = {"prefill_ms": round(t_pre * 1e3, 2), "prefill_tokens_per_s": round(batch * prompt / t_pre),
+                            "decode_ms_per_step": round(step * 1e3, 3),
+                            "decode_tokens_per_s": round(batch / step), "generate_1_ms": round(t_gen0 * 1e3, 2)}
+
+        torch.manual_seed(5)
+        with torch.device(dev):
+            model = LugitarLM(LugitarConfig.from_dict(_lugitar_config(width, heads, ff, layers))).to(torch.bfloat16).eval()
+        legs("lugitar_bf16", model)
+        del model
+        cfg = AutoRegressiveLMConfig(hidden_size=width, num_hidden_layers=layers, num_attention_heads=heads,
+                                     num_key_value_heads=heads // 4, intermediate_size=ff,
+                                     max_position_embeddings=prompt + 2 * steps)
+        with torch.device(dev):
+            model = AutoRegressiveLM(cfg).to(torch.bfloat16).eval()
+        legs("dense_bf16", model)
+        w8a8.int8_state().reset()
+        fuse_int8_weights(model)
+        with w8a8.int8_autocast(True):
+            legs("dense_fused_int8", model)
+        w8a8.int8_state().reset()
+        del model
+        torch.cuda.empty_cache()
+        out["models"].append(row)
+        print(json.dumps(row), file=sys.stderr, flush=True)
+    for width, heads, ff, batch, seq in ((2048, 16, 5632, 32, 512), (4096, 32, 8192, 4, 4096)):
+        k = {"width": width, "heads": heads, "ff": ff, "batch": batch, "seq": seq,
+             "kernels": _lugitar_kernels(dev, width, heads, ff, batch, seq)}
+        out["kernels"].append(k)
+        print(json.dumps(k), file=sys.stderr, flush=True)
+    return out
+
+
 def _cpu_decoder_baseline(layers=1, prefill_batch=8, decode_steps=8):
     """BASELINE config 4 on the host CPU through the decoder oracle (every Linear the exact
     int8 oracle, dense cache), on a bounded sample: a `layers`-layer model of the config-4
@@ -389,6 +563,12 @@ def main():
     ap.add_argument("--trace-gemms", action="store_true",
                     help="tracing mode: a few launches of the large GEMM kernels besides the headline one "
                          "(int8 4096^3, block-scaled config 3, fp8 with e4m3 output), nothing else")
+    ap.add_argument("--lugitar", action="store_true",
+                    help="Lugitar models beside the dense decoder of equal size (prompt and decode throughput) and "
+                         "every kernel of theirs beside the like kernel of the dense decoder, nothing else")
+    ap.add_argument("--lugitar-trace", action="store_true",
+                    help="tracing mode: an 8-layer Lugitar model, one 32 x 512-token prompt + 7 eager decode steps, "
+                         "nothing else")
     ap.add_argument("--pmc", action="store_true",
                     help="counter-collection mode: a few launches of the headline kernel and of a "
                          "plain 256 MiB device copy (the calibration kernel), nothing else")
@@ -397,7 +577,8 @@ def main():
         sys.exit("bench.py measures one GPU's share of the path: run with --gpus 1 "
                  "(no multi-GPU leg exists: the path shards by output columns or by K, one collective at most)")
 
-    tracing = bool(args.decoder_trace or args.trace_kernels or args.trace_gemms or args.pmc)
+    tracing = bool(args.decoder_trace or args.trace_kernels or args.trace_gemms or args.pmc or args.lugitar
+                   or args.lugitar_trace)
     ceilings = {} if tracing else _measured_ceilings()
 
     import torch
@@ -416,6 +597,21 @@ def main():
     def check(rc):
         if rc:
             raise RuntimeError(lib.astrai_w8a8_last_error().decode())
+
+    if args.lugitar:
+        print(json.dumps({"lugitar": _bench_lugitar(dev)}))
+        return
+    if args.lugitar_trace:
+        from astrai_amd.model import LugitarConfig, LugitarLM, greedy_generate
+
+        torch.manual_seed(5)
+        with torch.device(dev):
+            model = LugitarLM(LugitarConfig.from_dict(_lugitar_config(2048, 16, 5632, 8))).to(torch.bfloat16).eval()
+        ids = torch.randint(0, 32000, (32, 512), generator=torch.Generator().manual_seed(4)).to(dev)
+        greedy_generate(model, ids, 8)
+        torch.cuda.synchronize()
+        print(json.dumps({"lugitar_trace": "8 layers", "prompt_tokens": 32 * 512, "decode_steps": 7}))
+        return
 
     if args.decoder_trace:
         from astrai_amd.extension import w8a8

@@ -59,33 +59,34 @@ int astrai_mix_gated_rms_norm(const void* o, const void* g, int64_t ldg, const f
  * columns, at dkv_off (>= 0) the rp + dr latent columns. Rotates the first 2 * half of every head's dr
  * rotated columns in place (pairs i, i + half; rot [rot_rows, half, 2] = cos, sin per position),
  * writes (RMS norm of the latent over kv_rank columns, rotated key part) into
- * cache [batch, max_len, rp + dr] at positions [seq]. dkv_off < 0: queries only. */
+ * cache [batch, max_len, rp + dr] at positions [seq]. dkv_off < 0: queries only. With q_abs (bf16
+ * [batch * seq, heads, rp], else null): also q_abs = W_uk^T q_unrotated per head, w_uk_t
+ * [heads, rp, dn] being W_uk's rows transposed. */
 int astrai_mix_latent_append(void* proj, int64_t ld, int64_t dkv_off, const float* rot, int64_t rot_rows,
                              int64_t half, const int64_t* positions, const float* norm_w, void* cache,
-                             int64_t batch, int64_t seq, int64_t max_len, int64_t heads, int64_t dn,
-                             int64_t dr, int64_t rp, int64_t kv_rank, float eps, int dtype, void* stream);
+                             const void* w_uk_t, void* q_abs, int64_t batch, int64_t seq, int64_t max_len,
+                             int64_t heads, int64_t dn, int64_t dr, int64_t rp, int64_t kv_rank, float eps, int dtype, void* stream);
 
 /* Sliding-window attention of seq new tokens at positions start .. start + seq - 1 (bf16). kv
  * [batch, n_keys, heads * (dn + vp)]: per head the unrotated key and the value of positions
  * key_base .. ; the rotated key part comes from the cache. Query p sees keys p - window + 1 .. p.
  * Head h's output is multiplied by sigmoid(proj[:, g_off + h]). out [batch, seq, heads * vp].
- * UNSUPPORTED unless dn + dr <= 256 and vp <= 128. */
+ * UNSUPPORTED unless dn <= 128, dr <= 64, vp <= 128 and 1e-4 <= scale <= 1e4. */
 int astrai_mix_latent_prefill(const void* proj, int64_t ld, int64_t g_off, const void* kv, const void* cache,
                               void* out, int64_t batch, int64_t seq, int64_t max_len, int64_t start,
                               int64_t key_base, int64_t n_keys, int64_t heads, int64_t dn, int64_t dr,
                               int64_t rp, int64_t vp, int64_t window, float scale, void* stream);
 
-/* The same for a few new tokens, attending in the latent space (W_uk absorbed into the query,
- * W_uv applied to the attended latent): w_ukv [heads * (dn + vp), rp], per head the key rows then
- * the value rows; w_uk_t [heads, rp, dn] the transposed key rows. Positions come from the device.
- * nsplit workgroups share a context (1 .. ASTRAI_MIX_MAX_SPLIT). bf16; q_abs bf16
- * [batch * seq, heads, rp] and ws (astrai_mix_latent_rows_workspace_floats) are scratch.
- * UNSUPPORTED unless rp <= 1024 and rp + dr <= 1152. */
+/* The same for a few new tokens, attending in the latent space with the absorbed queries of
+ * latent_append; W_uv is applied to the attended latent. w_ukv [heads * (dn + vp), rp]: per head the key
+ * rows, then the value rows. Positions come from the device. nsplit workgroups share a context (1 ..
+ * ASTRAI_MIX_MAX_SPLIT). bf16; q_abs is overwritten, ws (astrai_mix_latent_rows_workspace_floats)
+ * scratch. UNSUPPORTED unless rp <= 1024, dr <= 64 and a sequence's cache stays below 2 GiB. */
 int64_t astrai_mix_latent_rows_workspace_floats(int64_t tokens, int64_t heads, int64_t rp, int64_t nsplit);
-int astrai_mix_latent_rows(const void* proj, int64_t ld, int64_t g_off, const void* w_ukv, const void* w_uk_t,
-                           const void* cache, const int64_t* positions, void* q_abs, float* ws, void* out,
-                           int64_t batch, int64_t seq, int64_t max_len, int64_t heads, int64_t dn, int64_t dr,
-                           int64_t rp, int64_t vp, int64_t window, float scale, int64_t nsplit, void* stream);
+int astrai_mix_latent_rows(const void* proj, int64_t ld, int64_t g_off, const void* w_ukv, const void* cache,
+                           const int64_t* positions, void* q_abs, float* ws, void* out, int64_t batch,
+                           int64_t seq, int64_t max_len, int64_t heads, int64_t dn, int64_t dr, int64_t rp,
+                           int64_t vp, int64_t window, float scale, int64_t nsplit, void* stream);
 
 /* The same arithmetic on the vector ALU, bf16 or float, rp <= 2048 and dr <= 512. */
 int astrai_mix_latent_rows_general(const void* proj, int64_t ld, int64_t g_off, const void* w_ukv,

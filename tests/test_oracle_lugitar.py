@@ -1,0 +1,327 @@
+"""The plain Lugitar implementation against what its equations fix, and the parts of the framework's
+Lugitar code that need no GPU."""
+
+import ctypes
+import json
+import math
+import os
+import re
+
+import pytest
+import torch
+
+import lugitar_helpers as H
+from astrai_amd.extension import _mix
+from astrai_amd.model import (LugitarConfig, LugitarLM, MixerCache, RequestCaches, StepCache, architecture_of,
+                              architectures, load_checkpoint)
+from astrai_amd.model.decoder import AutoRegressiveLM, AutoRegressiveLMConfig, yarn_frequencies
+from astrai_amd.model.mixers import PackedLinear, Rotation, Rows, heads_of
+from oracle import lugitar_oracle as L
+
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+
+
+# ---------------------------------------------------------------- the plain implementation
+
+
+def test_lightning_scan_is_the_decayed_sum():
+    g = torch.Generator().manual_seed(1)
+    q, k, v = (torch.randn(9, 2, n, generator=g, dtype=torch.float64) for n in (5, 5, 3))
+    decay = (0.7, 1.0)
+    out, state = L.lightning_scan(q, k, v, decay)
+    for h in range(2):
+        for t in range(9):
+            want = sum(decay[h] ** (t - j) * (q[t, h] @ k[j, h]) * v[j, h] for j in range(t + 1))
+            assert torch.allclose(out[t, h], want)
+        want = sum(decay[h] ** (8 - j) * torch.outer(k[j, h], v[j, h]) for j in range(9))
+        assert torch.allclose(state[h], want)
+    a, s = L.lightning_scan(q[:4], k[:4], v[:4], decay)
+    b, s = L.lightning_scan(q[4:], k[4:], v[4:], decay, s)
+    assert torch.allclose(torch.cat([a, b]), out) and torch.allclose(s, state)
+
+
+def test_norms():
+    x = torch.tensor([[3.0, -1.0, 2.0, 0.0]], dtype=torch.float64)
+    w = torch.tensor([1.0, 2.0, 1.0, 1.0], dtype=torch.float64)
+    y = L.layer_norm(x, w, 0.5)
+    assert torch.allclose(y, (x - 1.0) / math.sqrt((4 + 4 + 1 + 1) / 4 + 0.5) * w)
+    assert torch.allclose(L.rms_norm(x, w, 0.5), x / math.sqrt(14 / 4 + 0.5) * w)
+
+
+def test_window_mask_edges():
+    m = L.window_mask(6, 3)
+    assert m[4].tolist() == [False, False, True, True, True, False]
+    assert torch.equal(L.window_mask(6, 1), torch.eye(6, dtype=torch.bool))
+    assert torch.equal(L.window_mask(6, None), torch.ones(6, 6).tril().bool())
+
+
+def test_rotation_pairs_halves_and_leaves_the_rest():
+    x = torch.randn(3, 2, 10, dtype=torch.float64)
+    rot = H.rotation(6, base=50.0)
+    y = L.rotate_half(x, torch.tensor([0, 5, 9]), rot)
+    assert torch.allclose(y[0], x[0]) and torch.allclose(y[..., 6:], x[..., 6:])
+    a = 5 * 50.0 ** (-2 / 6)   # pair 1 at position 5
+    assert torch.allclose(y[1, :, 1], x[1, :, 1] * math.cos(a) - x[1, :, 4] * math.sin(a))
+    assert torch.allclose(y[1, :, 4], x[1, :, 4] * math.cos(a) + x[1, :, 1] * math.sin(a))
+
+
+def test_yarn_ends_and_middle():
+    dims, base, (factor, original, fast, slow) = 32, 1e4, (8.0, 4096, 32.0, 1.0)
+    rot = H.rotation(dims, base, (factor, original, fast, slow))
+    f, plain = L.rotary_frequencies(dims, base, rot["scaling"]), L.rotary_frequencies(dims, base, None)
+    assert f[0] == plain[0] and f[-1] == pytest.approx(plain[-1] / factor)   # fast pairs kept, slow ones stretched
+    lo = math.floor(dims * math.log(original / (2 * math.pi * fast)) / (2 * math.log(base)))
+    hi = math.ceil(dims * math.log(original / (2 * math.pi * slow)) / (2 * math.log(base)))
+    i = (lo + hi) // 2
+    ramp = (i - lo) / (hi - lo)
+    assert 0 < lo < i < hi < dims - 1
+    assert f[i] == pytest.approx(plain[i] * (ramp / factor + 1 - ramp))
+    assert L.rotary_magnitude(rot["scaling"]) == pytest.approx(0.1 * math.log(8.0) + 1)
+    # a window of turns that does not fit the dimensions is clamped at both ends
+    tiny = L.rotary_frequencies(8, 10.0, dict(factor=2.0, original=8, fast=1e6, slow=1e-6))
+    assert tiny[0] == pytest.approx(1.0) and tiny[3] == pytest.approx(10.0 ** (-6 / 8) * (3 / 7 / 2 + 4 / 7))
+
+
+def test_far_tokens_are_cut_off_by_the_window_and_kept_by_the_state():
+    one = H.config([H.latent(window=5)])
+    w = H.tensors(one, 3)
+    a = list(range(20))
+    b = [50] + a[1:]
+    la, lb = L.forward(one, w, a), L.forward(one, w, b)
+    assert not torch.allclose(la[4], lb[4]) and torch.equal(la[5:], lb[5:])
+    two = H.config([H.lightning()])
+    w = H.tensors(two, 3)
+    assert not torch.allclose(L.forward(two, w, a)[-1], L.forward(two, w, b)[-1])
+
+
+def test_shared_latents_come_from_the_named_layer():
+    cfg = H.config([H.latent(), H.latent(), H.latent(kv_from=0), H.latent(kv_from=1)])
+    w = H.tensors(cfg, 5)
+    base = L.forward(cfg, w, range(9))
+    # with the values of both sources swapped the result differs: the two are told apart
+    cfg2 = H.config([H.latent(), H.latent(), H.latent(kv_from=1), H.latent(kv_from=0)])
+    assert not torch.allclose(base, L.forward(cfg2, w, range(9)))
+
+
+# ---------------------------------------------------------------- framework parts on the CPU
+
+
+@pytest.mark.parametrize("dims,base,scaling", [(8, 500.0, H.YARN), (64, 1e4, (4.0, 4096, 32.0, 1.0)),
+                                                (6, 30.0, (2.0, 16, 1e5, 1e-5)), (2, 7.0, (3.0, 100, 2.0, 2.0))])
+def test_rotary_tables_agree_with_the_plain_rotation(dims, base, scaling):
+    rot = H.rotation(dims, base, scaling)
+    s = rot["scaling"]
+    f = yarn_frequencies(dims, base, s["factor"], s["original"], s["fast"], s["slow"])
+    assert torch.allclose(f, torch.tensor(L.rotary_frequencies(dims, base, s), dtype=torch.float64), rtol=1e-14)
+    table = Rotation.from_dict(rot).table(40)
+    x = torch.randn(40, dims, dtype=torch.float64)
+    y = L.rotate_half(x, torch.arange(40), rot)
+    u, v, cs = x[:, :dims // 2], x[:, dims // 2:], table.double()
+    z = torch.cat([u * cs[..., 0] - v * cs[..., 1], v * cs[..., 0] + u * cs[..., 1]], -1)
+    assert table.dtype == torch.float32 and torch.allclose(y, z, atol=1e-6)
+
+
+def test_packed_rows_and_columns_pad_with_zeros():
+    r = heads_of("q", 2, 3, 5)
+    assert r.size == 16 and r.padded == 128
+    t = torch.arange(16.0)
+    p = r.pack(t).reshape(2, 64)
+    assert p[1, :3].tolist() == [8, 9, 10] and p[1, 32:37].tolist() == [11, 12, 13, 14, 15]
+    assert p.count_nonzero() == 15
+    lin = PackedLinear(heads_of("h", 2, 5), [Rows("a", 1, ((4, 8),)), heads_of("b", 1, 3)])
+    lin.reset_parameters()
+    w = torch.randn(4, 10)
+    lin.assign("a", w)
+    assert lin.offset == {"a": 0, "b": 8} and lin.weight.shape == (40, 64)
+    assert torch.equal(lin.weight[:4, :5], w[:, :5]) and torch.equal(lin.weight[:4, 32:37], w[:, 5:])
+    assert lin.weight[4:8].count_nonzero() == 0 and lin.weight[:, 5:32].count_nonzero() == 0
+    assert lin.weight[8:11].count_nonzero() == 30 and lin.weight[11:].count_nonzero() == 0
+
+
+def test_registry_picks_the_classes_by_config():
+    assert {"Lugitar", "AutoRegressiveLM"} <= set(architectures())
+    arch = architecture_of(H.mixed())
+    assert arch.model_class is LugitarLM and isinstance(arch.make_config(H.mixed()), LugitarConfig)
+    dense = architecture_of({"vocab_size": 8})
+    assert dense.model_class is AutoRegressiveLM and dense.make_config({"vocab_size": 8}).vocab_size == 8
+    with pytest.raises(ValueError, match="unknown architecture 'Nope'"):
+        architecture_of({"architecture": "Nope"})
+
+
+def _save(tmp_path, cfg, tensors):
+    import safetensors.torch as st
+    (tmp_path / "config.json").write_text(json.dumps(cfg))
+    st.save_file(tensors, str(tmp_path / "model.safetensors"))
+    return str(tmp_path)
+
+
+def test_checkpoint_loading_takes_every_tensor(tmp_path):
+    cfg = H.mixed()
+    w = H.tensors(cfg, 2)
+    m = load_checkpoint(_save(tmp_path, cfg, w), "cpu", torch.bfloat16)
+    mix = m.layers[0].mix
+    assert torch.equal(mix.in_proj.weight[:24], w["l0.mix.q"][:24])
+    assert torch.equal(mix.in_proj.weight[32:40], w["l0.mix.q"][24:32])
+    assert torch.equal(m.layers[1].norm1.weight, w["l1.norm1"].float())
+    # decay powers and norm weights stay fp32 in a bf16 model
+    pw = m.layers[1].mix.decay.weight.view(3, -1)
+    assert pw.dtype == torch.float32 and pw[2, 64].item() == pytest.approx(0.9995 ** 64, rel=1e-7)
+    missing = {k: t for k, t in w.items() if k != "l3.mix.uv"}
+    with pytest.raises(ValueError, match="l3.mix.uv is missing"):
+        load_checkpoint(_save(tmp_path, cfg, missing), "cpu")
+    with pytest.raises(ValueError, match="unexpected .*l9.norm1"):
+        load_checkpoint(_save(tmp_path, cfg, {**w, "l9.norm1": w["l0.norm1"].clone()}), "cpu")
+    with pytest.raises(ValueError, match="l0.mix.o has shape"):
+        load_checkpoint(_save(tmp_path, cfg, {**w, "l0.mix.o": w["l0.mix.o"][:-1].clone()}), "cpu")
+
+
+def test_dense_checkpoint_loads_through_the_same_entry(tmp_path):
+    cfg = dict(vocab_size=32, hidden_size=16, num_hidden_layers=1, num_attention_heads=2, num_key_value_heads=1,
+               intermediate_size=24, max_position_embeddings=16)
+    torch.manual_seed(0)
+    model = AutoRegressiveLM(AutoRegressiveLMConfig(**cfg))
+    d = _save(tmp_path, cfg, {k: v.contiguous() for k, v in model.state_dict().items()})
+    got = load_checkpoint(d, "cpu", torch.float32)
+    ids = torch.arange(6).reshape(1, 6)
+    want = model(ids)["logits"]
+    assert torch.equal(got(ids)["logits"], want)
+    # the trace runner's step: portions through a cache, only the wanted places
+    from astrai_amd.trace import replay
+    caches = RequestCaches(lambda: got.new_cache(1, 6))
+    with torch.no_grad():
+        for n, (lo, hi) in enumerate(((0, 3), (3, 4), (4, 6))):
+            replay(got, caches, {"step": n, "entries": [{"id": "a", "tokens": list(range(lo, hi)), "want": [hi - lo - 1]}],
+                                 "end": []}, str(tmp_path))
+            rows = torch.frombuffer(bytearray((tmp_path / f"{n}.f32").read_bytes()), dtype=torch.float32)
+            assert torch.allclose(rows, want[0, hi - 1], atol=1e-5)
+
+
+def test_bad_layer_descriptions_are_refused():
+    def build(layers):
+        return LugitarLM(LugitarConfig.from_dict(H.config(layers)))
+    with pytest.raises(ValueError, match="kv_from 1 is not an earlier"):
+        build([H.latent(), H.lightning(), H.latent(kv_from=1)])
+    with pytest.raises(ValueError, match="has no latents of its own"):
+        build([H.latent(), H.latent(kv_from=0), H.latent(kv_from=1)])
+    with pytest.raises(ValueError, match="kv_rank differs"):
+        build([H.latent(), H.latent(kv_rank=48, kv_from=0)])
+    with pytest.raises(ValueError, match="2 decays for 3 heads"):
+        build([H.lightning(decay=(0.5, 0.6))])
+    with pytest.raises(ValueError, match="unknown mixer"):
+        build([dict(H.lightning(), type="other")])
+
+
+def test_caches_are_lent_reset_and_bounded():
+    made = []
+
+    def new():
+        c = MixerCache(1, 8, "cpu", torch.float32)
+        c.add_state(0, 2, 3)
+        made.append(c)
+        return c
+
+    pool = RequestCaches(new)
+    a, b = pool.of("a"), pool.of("b")
+    assert a is not b and pool.of("a") is a
+    assert a.next_positions(3).tolist() == [0, 1, 2]
+    a.advance(3)
+    a.state[0].fill_(1.0)
+    assert a.next_positions(2).tolist() == [3, 4]
+    with pytest.raises(ValueError, match="6 tokens after 3 do not fit"):
+        a.next_positions(6)
+    pool.end("a")
+    pool.end("unknown")
+    c = pool.of("c")
+    assert c is a and c.tokens == 0 and c.state[0].count_nonzero() == 0 and len(made) == 2
+    assert isinstance(c, StepCache)
+
+
+def test_decay_powers_cover_one_and_zero():
+    p = _mix.decay_powers([1.0, 0.0, 0.5])
+    assert p.shape == (3, _mix.LIGHTNING_CHUNK + 1) and p.dtype == torch.float32
+    assert p[0].eq(1).all() and p[1, 0] == 1 and p[1, 1:].eq(0).all() and p[2, 5] == 0.5 ** 5
+
+
+def test_launch_plans():
+    s = _mix.LatentShape(16, 128, 64, 512, 128, 512, 1024, 0.07)
+    assert _mix.latent_rows_nsplit(s, 32, 1, 1024) == 8      # 32 row tiles; four 32-key tiles a split
+    assert _mix.latent_rows_nsplit(s, 1, 1, 64) == 1
+    assert _mix.latent_rows_nsplit(s, 600, 1, 1 << 20) == 1
+    assert _mix.lightning_nseg(32, 16, 128, 512) == 1 and _mix.lightning_nseg(1, 16, 128, 4096) == 16
+    assert _mix.lightning_nseg(1, 4, 32, 70) == 1
+
+
+# ---------------------------------------------------------------- the C ABI without a GPU
+
+
+def _declared():
+    text = open(os.path.join(ROOT, "include", "astrai_mix.h")).read()
+    text = re.sub(r"/\*.*?\*/", "", text, flags=re.S)
+    return text, sorted(set(re.findall(r"\b(astrai_mix_[a-z0-9_]+)\s*\(", text)))
+
+
+def test_mix_header_library_and_binding_agree():
+    text, names = _declared()
+    assert names == sorted(_mix.PROTOTYPES)
+    assert os.path.exists(_mix.LIB_PATH), "build with `make -C astrai_amd/csrc mix`"
+    lib = ctypes.CDLL(_mix.LIB_PATH)
+    for name in names:
+        assert hasattr(lib, name), name
+        args = re.search(rf"\b{name}\s*\((.*?)\)\s*;", text, flags=re.S).group(1)
+        count = 0 if args.strip() == "void" else args.count(",") + 1
+        assert count == len(_mix.PROTOTYPES[name][0]), name
+    for macro, value in (("ABI_VERSION", _mix.ABI_VERSION), ("LIGHTNING_CHUNK", _mix.LIGHTNING_CHUNK),
+                         ("MAX_SPLIT", _mix.MAX_SPLIT)):
+        assert int(re.search(rf"#define ASTRAI_MIX_{macro}\s+(\d+)", text).group(1)) == value
+
+
+def test_mix_registry_names():
+    from astrai_amd.extension import KERNEL_NAMES, get_module, is_available
+    for name in ("latent_attention", "lightning_attention", "residual_rows"):
+        assert name in KERNEL_NAMES and is_available(name)
+    assert get_module("lightning_attention").lightning is _mix.lightning
+
+
+def test_mix_arguments_are_validated_before_anything_is_launched():
+    """16 stands for an aligned non-null pointer that is never dereferenced."""
+    lib = _mix.load()
+    assert lib is not None, _mix.load_error()
+    P = 16
+
+    def err():
+        return lib.astrai_mix_last_error().decode()
+
+    assert lib.astrai_mix_residual_norm(P, P, P, P, None, P, 4, 8, 1.0, 1e-6, 0, None) == 1 and "null" in err()
+    assert lib.astrai_mix_residual_norm(P, P, P, 8, P, P, 4, 8, 1.0, 1e-6, 0, None) == 1 and "aligned" in err()
+    assert lib.astrai_mix_residual_norm(P, P, P, P, P, P, 4, 8, 1.0, 1e-6, 7, None) == 1 and "dtype" in err()
+    assert lib.astrai_mix_silu_mul(P, P, 4, 12, 0, None) == 1
+    assert lib.astrai_mix_gated_rms_norm(P, P, 8, P, P, 4, 16, 16, 1e-6, 0, None) == 1
+    tail = (1, 8, 64, 3, 32, 32, 64, 56, 1e-6, 0, None)   # batch, seq, max_len, heads, dn, dr, rp, kv_rank
+    assert lib.astrai_mix_latent_append(P, 200, 192, P, 64, 4, P, P, P, None, None, *tail) == 1 and "row stride" in err()
+    bad = (1, 8, 64, 3, 40, 32, 64, 56, 1e-6, 0, None)
+    assert lib.astrai_mix_latent_append(P, 320, 192, P, 64, 4, P, P, P, None, None, *bad) == 1 and "multiples of 32" in err()
+    # keys that do not reach back a whole window, or not up to the newest token
+    dims = (3, 32, 32, 64, 64, 16, 0.5, None)             # heads, dn, dr, rp, vp, window, scale
+    assert lib.astrai_mix_latent_prefill(P, 320, 300, P, P, P, 1, 32, 100, 20, 6, 46, *dims) == 1 and "do not cover" in err()
+    assert lib.astrai_mix_latent_prefill(P, 320, 300, P, P, P, 1, 32, 100, 20, 5, 46, *dims) == 1 and "do not cover" in err()
+    wide = (3, 160, 32, 64, 64, 16, 0.5, None)
+    assert lib.astrai_mix_latent_prefill(P, 640, 600, P, P, P, 1, 32, 100, 20, 5, 47, *wide) == 2
+    assert not _mix.latent_prefill_supported(_mix.LatentShape(3, 160, 32, 64, 64, 64, 16, 0.5))
+    rows = (P, 320, 300, P, P, P, P, P, P, 1, 2, 100)
+    assert lib.astrai_mix_latent_rows(*rows, 3, 32, 32, 1056, 64, 16, 0.5, 1, None) == 2
+    assert not _mix.latent_rows_supported(_mix.LatentShape(3, 32, 32, 1056, 64, 1056, 16, 0.5), 100)
+    assert lib.astrai_mix_latent_rows(*rows, 3, 32, 32, 64, 64, 16, 0.5, 65, None) == 1 and "nsplit" in err()
+    assert lib.astrai_mix_latent_rows_general(P, 320, 300, P, P, P, P, 1, 2, 100, 3, 32, 32, 4096, 64, 16, 0.5, 1, None) == 2
+    lt = (P, 320, 0, 96, 192, P, P)
+    assert lib.astrai_mix_lightning_chunk(*lt, None, P, 1, 70, 3, 32, 32, 3, None) == 1 and "nseg" in err()
+    assert lib.astrai_mix_lightning_chunk(*lt, None, P, 1, 70, 3, 32, 32, 2, None) == 1 and "nseg" in err()
+    assert lib.astrai_mix_lightning_step(*lt, P, 1, 70, 5, 32, 32, 0, None) == 1 and "do not fit" in err()
+    assert lib.astrai_mix_lightning_chunk(P, 4096, 0, 288, 576, P, P, None, P, 1, 70, 1, 288, 32, 1, None) == 2
+
+
+def test_trace_runner_reads_its_arguments(capsys):
+    from astrai_amd import trace
+    with pytest.raises(SystemExit):
+        trace.main(["--dtype", "int4"])
+    assert "--max-tokens" in capsys.readouterr().err
+    assert os.access(os.path.join(ROOT, "bin", "trace_run"), os.X_OK)
