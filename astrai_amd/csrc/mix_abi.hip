@@ -10,6 +10,8 @@
 #include "mix_launchers.h"
 
 static_assert(astrai_mix::kMaxSplit == ASTRAI_MIX_MAX_SPLIT && astrai_mix::kLightningChunk == ASTRAI_MIX_LIGHTNING_CHUNK);
+static_assert(astrai_mix::kRingSteps == ASTRAI_MIX_RING_STEPS && astrai_mix::kDeltaChunk == ASTRAI_MIX_DELTA_CHUNK);
+static_assert(astrai_mix::kActSilu == ASTRAI_MIX_SILU && astrai_mix::kActGelu == ASTRAI_MIX_GELU);
 
 namespace {
 
@@ -120,13 +122,89 @@ LightningArgs lightning_args(const void* proj, int64_t ld, int64_t q_off, int64_
     return a;
 }
 
-}  // namespace
-
 #define MIX_TRY(expr)                     \
     do {                                  \
         const int rc_ = (expr);           \
         if (rc_ != ASTRAI_MIX_OK) return rc_; \
     } while (0)
+
+int check_gqa(const char* what, int64_t heads, int64_t kv_heads, int64_t dk, int64_t vp) {
+    if (heads <= 0 || kv_heads <= 0 || heads % kv_heads || heads > kMaxGridYZ || !pad32(dk, 32) || !pad32(vp, 32) ||
+        heads * dk > kMaxInt || heads * vp > kMaxInt || kv_heads * (dk + vp) > kMaxInt)
+        return fail(ASTRAI_MIX_BAD_ARG, "%s: bad heads %lld / %lld or head sizes %lld, %lld (positive multiples of 32)", what,
+                    (long long)heads, (long long)kv_heads, (long long)dk, (long long)vp);
+    return ASTRAI_MIX_OK;
+}
+
+int check_gate(const char* what, int64_t ld, int64_t g_off, int64_t cols) {
+    if (g_off >= 0 && (g_off % 8 || g_off + cols > ld)) return fail(ASTRAI_MIX_BAD_ARG, "%s: bad gate columns", what);
+    return ASTRAI_MIX_OK;
+}
+
+GqaDims gqa_dims(int64_t heads, int64_t kv_heads, int64_t dk, int64_t vp, int64_t window, float scale, float softcap,
+                 int sink) {
+    return GqaDims{(int)heads, (int)kv_heads, (int)dk, (int)vp, window_of(window), scale, softcap, sink};
+}
+
+int check_conv(const char* what, int64_t ld, int64_t off, int64_t cols, const float* w, const float* bias, int64_t taps,
+               const void* ring, const int64_t* positions) {
+    MIX_TRY(check_ptrs(what, (const void*)w, ring));
+    if (!positions) return fail(ASTRAI_MIX_BAD_ARG, "%s: null pointer", what);
+    if (bias) MIX_TRY(check_ptrs(what, (const void*)bias));
+    if (taps < 1 || taps > 1024 || cols <= 0 || cols % 4 || off < 0 || off % 4 || off + cols > ld)
+        return fail(ASTRAI_MIX_BAD_ARG, "%s: bad columns %lld .. + %lld of %lld or taps %lld", what, (long long)off,
+                    (long long)cols, (long long)ld, (long long)taps);
+    return ASTRAI_MIX_OK;
+}
+
+ConvArgs conv_args(const void* proj, int64_t ld, int64_t off, int64_t cols, const float* w, const float* bias, int64_t taps,
+                   void* ring, const int64_t* positions, void* out, int64_t batch, int64_t seq, int silu) {
+    return ConvArgs{proj, ld, (int)off, (int)cols, w, bias, ring, positions, out, (int)batch, (int)seq, (int)taps,
+                    (int)taps - 1 + kRingSteps, silu};
+}
+
+int check_rglru(const char* what, int64_t ld, int64_t y_off, int64_t batch, int64_t seq, int64_t blocks, int64_t bp) {
+    MIX_TRY(check_block(what, batch, seq, seq, ld, 8));
+    if (blocks <= 0 || !pad32(bp, 32) || blocks * bp > kMaxInt / 64 || y_off < 0 || y_off % 4 || y_off + blocks * bp > ld)
+        return fail(ASTRAI_MIX_BAD_ARG, "%s: bad blocks %lld x %lld (a multiple of 32) or columns", what, (long long)blocks,
+                    (long long)bp);
+    return ASTRAI_MIX_OK;
+}
+
+RglruArgs rglru_args(const void* u, const void* proj, int64_t ld, int64_t y_off, const void* w_r,
+                     const void* w_i, const float* b_r, const float* b_i, const float* coef, float* state, float* scratch,
+                     void* out, int64_t batch, int64_t seq, int64_t blocks, int64_t bp, int64_t nseg) {
+    RglruArgs a = {};
+    a.proj = proj;
+    a.ld = ld;
+    a.y_off = (int)y_off;
+    a.u = u;
+    a.w_r = w_r;
+    a.w_i = w_i;
+    a.b_r = b_r;
+    a.b_i = b_i;
+    a.coef = coef;
+    a.state = state;
+    a.scratch = scratch;
+    a.out = out;
+    a.batch = (int)batch;
+    a.seq = (int)seq;
+    a.blocks = (int)blocks;
+    a.bp = (int)bp;
+    a.nseg = (int)nseg;
+    return a;
+}
+
+int check_delta(const char* what, int64_t ld, int64_t b_off, int64_t batch, int64_t seq, int64_t heads, int64_t kv_heads,
+                int64_t dp, int64_t vp) {
+    MIX_TRY(check_gqa(what, heads, kv_heads, dp, vp));
+    MIX_TRY(check_block(what, batch, seq, seq, ld, 8));
+    if (b_off < 0 || b_off + heads > ld || 2 * kv_heads * dp + heads * vp > kMaxInt)
+        return fail(ASTRAI_MIX_BAD_ARG, "%s: bad step-size columns", what);
+    return ASTRAI_MIX_OK;
+}
+
+}  // namespace
 
 extern "C" {
 
@@ -161,14 +239,47 @@ int astrai_mix_embed_norm(const void* table, const int64_t* tokens, float* x_out
     return check_launch("embed_norm");
 }
 
-int astrai_mix_silu_mul(const void* gu, void* h, int64_t rows, int64_t ff, int dtype, void* stream) {
-    MIX_TRY(check_dtype("silu_mul", dtype));
-    MIX_TRY(check_ptrs("silu_mul", gu, (const void*)h));
-    if (rows < 0 || ff <= 0 || ff % 8 || ff > (1 << 24))
-        return fail(ASTRAI_MIX_BAD_ARG, "silu_mul: bad size %lld x %lld", (long long)rows, (long long)ff);
+int astrai_mix_sum_norm(const void* y, int64_t ldy, const int64_t* tokens, int64_t vocab, float mult, const float* x_in,
+                        const void* u, int64_t ldu, const float* vec, float* x_out, const float* w, void* h,
+                        int64_t rows, int64_t width, float eps, int y_float, int dtype, void* stream) {
+    MIX_TRY(check_dtype("sum_norm", dtype));
+    MIX_TRY(check_ptrs("sum_norm", y, (const void*)x_out, (const void*)h));
+    if (x_in) MIX_TRY(check_ptrs("sum_norm", (const void*)x_in));
+    if (u) MIX_TRY(check_ptrs("sum_norm", u));
+    if (vec) MIX_TRY(check_ptrs("sum_norm", (const void*)vec));
+    if (w) MIX_TRY(check_ptrs("sum_norm", (const void*)w));
+    if (rows < 0 || rows > kMaxInt || width <= 0 || width > (1 << 24) || ldy < width || (u && ldu < width) ||
+        (tokens && vocab <= 0))
+        return fail(ASTRAI_MIX_BAD_ARG, "sum_norm: bad size %lld x %lld (strides %lld, %lld)", (long long)rows,
+                    (long long)width, (long long)ldy, (long long)ldu);
     if (rows == 0) return ASTRAI_MIX_OK;
-    launch_silu_mul(gu, h, rows, (int)ff, dtype, static_cast<hipStream_t>(stream));
-    return check_launch("silu_mul");
+    const SumNormArgs a = {y, ldy, tokens, x_in, u, u ? ldu : 0, vec, x_out, w, h, rows, vocab, (int)width, mult, eps};
+    launch_sum_norm(a, dtype, y_float != 0, static_cast<hipStream_t>(stream));
+    return check_launch("sum_norm");
+}
+
+int astrai_mix_act_mul(const void* gu, void* h, int64_t rows, int64_t ff, int act, int dtype, void* stream) {
+    MIX_TRY(check_dtype("act_mul", dtype));
+    MIX_TRY(check_ptrs("act_mul", gu, (const void*)h));
+    if (rows < 0 || ff <= 0 || ff % 8 || ff > (1 << 24) || (act != ASTRAI_MIX_SILU && act != ASTRAI_MIX_GELU))
+        return fail(ASTRAI_MIX_BAD_ARG, "act_mul: bad size %lld x %lld or activation %d", (long long)rows, (long long)ff, act);
+    if (rows == 0) return ASTRAI_MIX_OK;
+    launch_act_mul(gu, h, rows, (int)ff, act, dtype, static_cast<hipStream_t>(stream));
+    return check_launch("act_mul");
+}
+
+int astrai_mix_head_gated_rms_norm(const void* o, const void* g, int64_t ldg, const float* w, void* out, int64_t rows,
+                                   int64_t heads, int64_t vp, int64_t count, float eps, int dtype, void* stream) {
+    MIX_TRY(check_dtype("head_gated_rms_norm", dtype));
+    MIX_TRY(check_ptrs("head_gated_rms_norm", o, g, (const void*)w, (const void*)out));
+    if (rows < 0 || heads <= 0 || vp <= 0 || vp % 4 || vp > (1 << 20) || rows * heads > kMaxInt || ldg % 4 ||
+        ldg < heads * vp || count <= 0 || count > vp)
+        return fail(ASTRAI_MIX_BAD_ARG, "head_gated_rms_norm: bad size %lld x %lld x %lld (%lld counted, stride %lld)",
+                    (long long)rows, (long long)heads, (long long)vp, (long long)count, (long long)ldg);
+    if (rows == 0) return ASTRAI_MIX_OK;
+    const HeadNormArgs a = {o, g, ldg, w, out, rows, (int)heads, (int)vp, (int)count, eps};
+    launch_head_gated_rms_norm(a, dtype, static_cast<hipStream_t>(stream));
+    return check_launch("head_gated_rms_norm");
 }
 
 int astrai_mix_gated_rms_norm(const void* o, const void* g, int64_t ldg, const float* w, void* out, int64_t rows,
@@ -331,6 +442,251 @@ int astrai_mix_lightning_step(const void* proj, int64_t ld, int64_t q_off, int64
     launch_lightning_step(lightning_args(proj, ld, q_off, k_off, v_off, decay_pow, state, nullptr, out, batch, seq,
                                          heads, dp, vp, 1), dtype, static_cast<hipStream_t>(stream));
     return check_launch("lightning_step");
+}
+
+int astrai_mix_gqa_append(void* proj, int64_t ld, int64_t k_off, int64_t v_off, const float* rot, int64_t rot_rows,
+                          int64_t half, const int64_t* positions, const float* q_norm, const float* k_norm,
+                          void* cache, int64_t batch, int64_t seq, int64_t max_len, int64_t heads, int64_t kv_heads,
+                          int64_t dk, int64_t vp, int64_t dim, float eps, int dtype, void* stream) {
+    MIX_TRY(check_dtype("gqa_append", dtype));
+    MIX_TRY(check_ptrs("gqa_append", (const void*)proj, (const void*)cache));
+    if (!positions) return fail(ASTRAI_MIX_BAD_ARG, "gqa_append: null pointer");
+    MIX_TRY(check_gqa("gqa_append", heads, kv_heads, dk, vp));
+    MIX_TRY(check_block("gqa_append", batch, seq, max_len, ld, heads * dk));
+    if (rot) MIX_TRY(check_ptrs("gqa_append", (const void*)rot));
+    if ((q_norm == nullptr) != (k_norm == nullptr)) return fail(ASTRAI_MIX_BAD_ARG, "gqa_append: one norm weight");
+    if (q_norm) MIX_TRY(check_ptrs("gqa_append", (const void*)q_norm, (const void*)k_norm));
+    if (k_off < heads * dk || v_off < heads * dk || k_off % 8 || v_off % 8 || k_off + kv_heads * dk > ld ||
+        v_off + kv_heads * vp > ld || dim <= 0 || dim > dk || (rot && (half <= 0 || 2 * half > dim || rot_rows <= 0)) ||
+        batch * seq * (heads + 2 * kv_heads) > kMaxInt)
+        return fail(ASTRAI_MIX_BAD_ARG, "gqa_append: bad columns (k %lld, v %lld, half %lld, dim %lld)", (long long)k_off,
+                    (long long)v_off, (long long)half, (long long)dim);
+    if (dk > 512 || vp > 512) return fail(ASTRAI_MIX_UNSUPPORTED, "gqa_append: head sizes %lld, %lld (at most 512)",
+                                          (long long)dk, (long long)vp);
+    const GqaAppendArgs a = {proj, ld, (int)k_off, (int)v_off, rot, positions, q_norm, k_norm, cache, batch * seq, rot_rows,
+                             (int)seq, (int)max_len, (int)half, (int)dim, eps};
+    launch_gqa_append(a, gqa_dims(heads, kv_heads, dk, vp, 1, 1.0f, 0.0f, 0), dtype, static_cast<hipStream_t>(stream));
+    return check_launch("gqa_append");
+}
+
+int astrai_mix_gqa_prefill(const void* proj, int64_t ld, int64_t g_off, const void* cache, void* out, int64_t batch,
+                           int64_t seq, int64_t max_len, int64_t start, int64_t heads, int64_t kv_heads, int64_t dk,
+                           int64_t vp, int64_t window, float scale, float softcap, int sink, void* stream) {
+    MIX_TRY(check_ptrs("gqa_prefill", proj, cache, (const void*)out));
+    MIX_TRY(check_gqa("gqa_prefill", heads, kv_heads, dk, vp));
+    MIX_TRY(check_block("gqa_prefill", batch, seq, max_len, ld, heads * dk));
+    MIX_TRY(check_gate("gqa_prefill", ld, g_off, heads * vp));
+    if (window <= 0 || start < 0 || start + seq > max_len)
+        return fail(ASTRAI_MIX_BAD_ARG, "gqa_prefill: tokens %lld .. %lld of %lld, window %lld", (long long)start,
+                    (long long)(start + seq - 1), (long long)max_len, (long long)window);
+    const LatentDims d = dims(heads, dk, 0, 32, vp, window, scale);
+    if (!gqa_prefill_supported(d) || ((seq + 127) / 128) * batch * heads > kMaxInt)
+        return fail(ASTRAI_MIX_UNSUPPORTED, "gqa_prefill: head sizes %lld, %lld (at most 128) or scale %g", (long long)dk,
+                    (long long)vp, (double)scale);
+    LatentPrefillArgs a;
+    a.proj = proj;
+    a.ld = ld;
+    a.g_off = g_off < 0 ? -1 : (int)g_off;
+    a.kv = a.cache = cache;
+    a.out = out;
+    a.batch = (int)batch;
+    a.seq = (int)seq;
+    a.max_len = a.n_keys = (int)max_len;
+    a.start = (int)start;
+    a.key_base = 0;
+    a.group = (int)(heads / kv_heads);
+    a.softcap = softcap;
+    a.sink = sink;
+    launch_gqa_prefill(a, d, static_cast<hipStream_t>(stream));
+    return check_launch("gqa_prefill");
+}
+
+int64_t astrai_mix_gqa_rows_workspace_floats(int64_t tokens, int64_t heads, int64_t vp, int64_t nsplit) {
+    return gqa_rows_workspace_floats(gqa_dims(heads, heads, 32, vp, 1, 1.0f, 0.0f, 0), tokens, (int)nsplit);
+}
+
+int astrai_mix_gqa_rows(const void* proj, int64_t ld, int64_t g_off, const void* cache, const int64_t* positions,
+                        float* ws, void* out, int64_t batch, int64_t seq, int64_t max_len, int64_t heads,
+                        int64_t kv_heads, int64_t dk, int64_t vp, int64_t window, float scale, float softcap, int sink,
+                        int64_t nsplit, void* stream) {
+    MIX_TRY(check_ptrs("gqa_rows", proj, cache, (const void*)ws, (const void*)out));
+    if (!positions) return fail(ASTRAI_MIX_BAD_ARG, "gqa_rows: null pointer");
+    MIX_TRY(check_gqa("gqa_rows", heads, kv_heads, dk, vp));
+    MIX_TRY(check_block("gqa_rows", batch, seq, max_len, ld, heads * dk));
+    MIX_TRY(check_gate("gqa_rows", ld, g_off, heads * vp));
+    if (window <= 0 || nsplit < 1 || nsplit > kMaxSplit)
+        return fail(ASTRAI_MIX_BAD_ARG, "gqa_rows: bad window or nsplit %lld", (long long)nsplit);
+    const GqaDims d = gqa_dims(heads, kv_heads, dk, vp, window, scale, softcap, sink);
+    if (!gqa_rows_mfma_supported(d) || seq * (heads / kv_heads) * nsplit > kMaxInt ||
+        (max_len + 64) * kv_heads * (dk + vp) * 2 >= kMaxInt)
+        return fail(ASTRAI_MIX_UNSUPPORTED, "gqa_rows: head sizes %lld, %lld (at most 256, 128), too many rows or a sequence of "
+                    "2 GiB", (long long)dk, (long long)vp);
+    const GqaRowsArgs a = {proj, ld, g_off < 0 ? -1 : (int)g_off, cache, positions, ws, out, (int)batch, (int)seq,
+                           (int)max_len, (int)nsplit};
+    launch_gqa_rows_mfma(a, d, static_cast<hipStream_t>(stream));
+    return check_launch("gqa_rows");
+}
+
+int astrai_mix_gqa_rows_general(const void* proj, int64_t ld, int64_t g_off, const void* cache,
+                                const int64_t* positions, void* out, int64_t batch, int64_t seq, int64_t max_len,
+                                int64_t heads, int64_t kv_heads, int64_t dk, int64_t vp, int64_t window, float scale,
+                                float softcap, int sink, int dtype, void* stream) {
+    MIX_TRY(check_dtype("gqa_rows_general", dtype));
+    MIX_TRY(check_ptrs("gqa_rows_general", proj, cache, (const void*)out));
+    if (!positions) return fail(ASTRAI_MIX_BAD_ARG, "gqa_rows_general: null pointer");
+    MIX_TRY(check_gqa("gqa_rows_general", heads, kv_heads, dk, vp));
+    MIX_TRY(check_block("gqa_rows_general", batch, seq, max_len, ld, heads * dk));
+    MIX_TRY(check_gate("gqa_rows_general", ld, g_off, heads * vp));
+    if (window <= 0) return fail(ASTRAI_MIX_BAD_ARG, "gqa_rows_general: bad window");
+    const GqaDims d = gqa_dims(heads, kv_heads, dk, vp, window, scale, softcap, sink);
+    if (!gqa_rows_general_supported(d))
+        return fail(ASTRAI_MIX_UNSUPPORTED, "gqa_rows_general: head sizes %lld, %lld (at most 1024)", (long long)dk, (long long)vp);
+    const GqaRowsArgs a = {proj, ld, g_off < 0 ? -1 : (int)g_off, cache, positions, nullptr, out, (int)batch, (int)seq,
+                           (int)max_len, 1};
+    launch_gqa_rows_general(a, d, dtype, static_cast<hipStream_t>(stream));
+    return check_launch("gqa_rows_general");
+}
+
+int astrai_mix_conv(const void* proj, int64_t ld, int64_t off, int64_t cols, const float* w, const float* bias,
+                    int64_t taps, void* ring, const int64_t* positions, void* out, int64_t batch, int64_t seq, int silu,
+                    int tail, int dtype, void* stream) {
+    MIX_TRY(check_dtype("conv", dtype));
+    MIX_TRY(check_ptrs("conv", proj));
+    if (out) MIX_TRY(check_ptrs("conv", (const void*)out));
+    MIX_TRY(check_block("conv", batch, seq, seq, ld, 8));
+    MIX_TRY(check_conv("conv", ld, off, cols, w, bias, taps, ring, positions));
+    if (batch * seq * (cols / 4) > (int64_t)kMaxInt * 64) return fail(ASTRAI_MIX_BAD_ARG, "conv: too many elements");
+    const ConvArgs a = conv_args(proj, ld, off, cols, w, bias, taps, ring, positions, out, batch, seq, silu);
+    if (out) launch_conv(a, dtype, static_cast<hipStream_t>(stream));
+    if (tail) launch_conv_tail(a, dtype, static_cast<hipStream_t>(stream));
+    return check_launch("conv");
+}
+
+int astrai_mix_rglru_chunk(const void* u, const void* proj, int64_t ld, int64_t y_off, const void* w_r, const void* w_i,
+                           const float* b_r, const float* b_i, const float* coef, float* state, float* scratch,
+                           void* out, int64_t batch, int64_t seq, int64_t blocks, int64_t bp, int64_t nseg,
+                           void* stream) {
+    MIX_TRY(check_ptrs("rglru_chunk", u, proj, w_r, w_i, (const void*)b_r, (const void*)b_i, (const void*)coef,
+                       (const void*)state, (const void*)out));
+    MIX_TRY(check_rglru("rglru_chunk", ld, y_off, batch, seq, blocks, bp));
+    if (nseg < 1 || nseg > seq || (nseg > 1 && !scratch) || blocks * ((bp + 63) / 64) > kMaxGridYZ)
+        return fail(ASTRAI_MIX_BAD_ARG, "rglru_chunk: bad nseg %lld or too many blocks", (long long)nseg);
+    if (!rglru_chunk_supported((int)bp))
+        return fail(ASTRAI_MIX_UNSUPPORTED, "rglru_chunk: blocks of %lld (at most 1024)", (long long)bp);
+    launch_rglru_chunk(rglru_args(u, proj, ld, y_off, w_r, w_i, b_r, b_i, coef, state, scratch, out, batch, seq, blocks,
+                                  bp, nseg), static_cast<hipStream_t>(stream));
+    return check_launch("rglru_chunk");
+}
+
+int astrai_mix_rglru_general(const void* u, const void* proj, int64_t ld, int64_t y_off, const void* w_r,
+                             const void* w_i, const float* b_r, const float* b_i, const float* coef, float* state,
+                             float* scratch, void* out, int64_t batch, int64_t seq, int64_t blocks, int64_t bp,
+                             int dtype, void* stream) {
+    MIX_TRY(check_dtype("rglru_general", dtype));
+    MIX_TRY(check_ptrs("rglru_general", u, proj, w_r, w_i, (const void*)b_r, (const void*)b_i, (const void*)coef,
+                       (const void*)state, (const void*)scratch, (const void*)out));
+    MIX_TRY(check_rglru("rglru_general", ld, y_off, batch, seq, blocks, bp));
+    if (batch * seq * blocks * bp > (int64_t)kMaxInt * 256) return fail(ASTRAI_MIX_BAD_ARG, "rglru_general: too many elements");
+    launch_rglru_general(rglru_args(u, proj, ld, y_off, w_r, w_i, b_r, b_i, coef, state, scratch, out, batch, seq,
+                                    blocks, bp, 1), dtype, static_cast<hipStream_t>(stream));
+    return check_launch("rglru_general");
+}
+
+int astrai_mix_rglru_step(const void* proj, int64_t ld, int64_t y_off, int64_t x_off, const float* conv_w,
+                          const float* conv_b, int64_t taps, void* ring, const int64_t* positions, const void* w_r,
+                          const void* w_i, const float* b_r, const float* b_i, const float* coef, float* state,
+                          void* out, int64_t batch, int64_t seq, int64_t blocks, int64_t bp, void* stream) {
+    MIX_TRY(check_ptrs("rglru_step", proj, w_r, w_i, (const void*)b_r, (const void*)b_i, (const void*)coef,
+                       (const void*)state, (const void*)out));
+    MIX_TRY(check_rglru("rglru_step", ld, y_off, batch, seq, blocks, bp));
+    MIX_TRY(check_conv("rglru_step", ld, x_off, blocks * bp, conv_w, conv_b, taps, ring, positions));
+    if (!rglru_step_supported((int)bp, (int)seq))
+        return fail(ASTRAI_MIX_UNSUPPORTED, "rglru_step: %lld tokens (at most %d)", (long long)seq, kRingSteps);
+    RglruArgs a = rglru_args(nullptr, proj, ld, y_off, w_r, w_i, b_r, b_i, coef, state, nullptr, out, batch, seq,
+                             blocks, bp, 1);
+    a.conv = conv_args(proj, ld, x_off, blocks * bp, conv_w, conv_b, taps, ring, positions, nullptr, batch, seq, 0);
+    launch_rglru_step(a, static_cast<hipStream_t>(stream));
+    return check_launch("rglru_step");
+}
+
+int astrai_mix_delta_step(const void* qkv, const void* proj, int64_t ld, int64_t x_off, int64_t b_off,
+                          const float* conv_w, int64_t taps, void* ring, const int64_t* positions, const float* z,
+                          const float* dt_bias, const float* decay, const void* gate, int64_t ldg, const float* norm_w,
+                          float* state, void* out, int64_t batch, int64_t seq, int64_t heads, int64_t kv_heads,
+                          int64_t dp, int64_t vp, int64_t vdim, float q_scale, float eps, int dtype, void* stream) {
+    MIX_TRY(check_dtype("delta_step", dtype));
+    MIX_TRY(check_ptrs("delta_step", proj, (const void*)z, (const void*)dt_bias, (const void*)decay, gate,
+                       (const void*)norm_w, (const void*)state, (const void*)out));
+    MIX_TRY(check_delta("delta_step", ld, b_off, batch, seq, heads, kv_heads, dp, vp));
+    const int64_t cols = 2 * kv_heads * dp + heads * vp;
+    if (qkv) MIX_TRY(check_ptrs("delta_step", qkv));
+    else MIX_TRY(check_conv("delta_step", ld, x_off, cols, conv_w, nullptr, taps, ring, positions));
+    if (ldg % 4 || ldg < heads * vp || vdim <= 0 || vdim > vp)
+        return fail(ASTRAI_MIX_BAD_ARG, "delta_step: bad gate stride %lld or value size %lld", (long long)ldg, (long long)vdim);
+    if (!delta_step_supported((int)dp, (int)vp) || (!qkv && seq > kRingSteps))
+        return fail(ASTRAI_MIX_UNSUPPORTED, "delta_step: head sizes %lld, %lld or %lld tokens", (long long)dp, (long long)vp,
+                    (long long)seq);
+    DeltaArgs a = {};
+    a.qkv = qkv;
+    a.ldq = cols;
+    a.proj = proj;
+    a.ld = ld;
+    a.b_off = (int)b_off;
+    a.z = z;
+    a.dt_bias = dt_bias;
+    a.decay = decay;
+    a.gate = gate;
+    a.ldg = ldg;
+    a.norm_w = norm_w;
+    a.state = state;
+    a.out = out;
+    a.batch = (int)batch;
+    a.seq = (int)seq;
+    a.heads = (int)heads;
+    a.kv_heads = (int)kv_heads;
+    a.dp = (int)dp;
+    a.vp = (int)vp;
+    a.vdim = (int)vdim;
+    a.q_scale = q_scale;
+    a.eps = eps;
+    if (!qkv) a.conv = conv_args(proj, ld, x_off, cols, conv_w, nullptr, taps, ring, positions, nullptr, batch, seq, 1);
+    launch_delta_step(a, !qkv, dtype, static_cast<hipStream_t>(stream));
+    return check_launch("delta_step");
+}
+
+int64_t astrai_mix_delta_image_bytes(int64_t dp) { return dp > 0 && dp <= 256 ? delta_image_bytes((int)dp) : 0; }
+
+int astrai_mix_delta_chunk(const void* qkv, const void* proj, int64_t ld, int64_t b_off, const float* z,
+                           const float* dt_bias, const float* decay, float* state, void* image, void* out, int64_t batch,
+                           int64_t seq, int64_t heads, int64_t kv_heads, int64_t dp, int64_t vp, float q_scale,
+                           void* stream) {
+    MIX_TRY(check_ptrs("delta_chunk", qkv, proj, (const void*)z, (const void*)dt_bias, (const void*)decay,
+                       (const void*)state, (const void*)image, (const void*)out));
+    MIX_TRY(check_delta("delta_chunk", ld, b_off, batch, seq, heads, kv_heads, dp, vp));
+    if (batch > kMaxGridYZ) return fail(ASTRAI_MIX_BAD_ARG, "delta_chunk: batch %lld", (long long)batch);
+    if (!delta_chunk_supported((int)dp, (int)vp))
+        return fail(ASTRAI_MIX_UNSUPPORTED, "delta_chunk: head size %lld (at most 256)", (long long)dp);
+    DeltaArgs a = {};
+    a.qkv = qkv;
+    a.ldq = 2 * kv_heads * dp + heads * vp;
+    a.proj = proj;
+    a.ld = ld;
+    a.b_off = (int)b_off;
+    a.z = z;
+    a.dt_bias = dt_bias;
+    a.decay = decay;
+    a.state = state;
+    a.image = image;
+    a.out = out;
+    a.batch = (int)batch;
+    a.seq = (int)seq;
+    a.heads = (int)heads;
+    a.kv_heads = (int)kv_heads;
+    a.dp = (int)dp;
+    a.vp = (int)vp;
+    a.q_scale = q_scale;
+    launch_delta_chunk(a, static_cast<hipStream_t>(stream));
+    return check_launch("delta_chunk");
 }
 
 }  // extern "C"

@@ -65,6 +65,53 @@ __device__ __forceinline__ float silu_as(float z) {
     return sizeof(T) == 2 ? silu_fast(z) : silu(z);
 }
 
+// tanh as 1 - 2 / (1 + e^(2z)), absolute error about 1e-7; e^(2z) may overflow or vanish
+__device__ __forceinline__ float tanh_fast(float z) {
+    return 1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(2.0f * kLog2e * z));
+}
+
+__device__ __forceinline__ float sigmoid_fast(float z) {
+    return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-kLog2e * z));
+}
+
+// gelu in its tanh form, z / 2 (1 + tanh(y)) = z sigmoid(2 y), y = sqrt(2 / pi) (z + 0.044715 z^3)
+template <typename T>
+__device__ __forceinline__ float gelu_as(float z) {
+    const float y2 = 1.5957691216057308f * (z + 0.044715f * z * z * z);
+    return z * (sizeof(T) == 2 ? sigmoid_fast(y2) : sigmoid(y2));
+}
+
+// 1 - e^x for x <= 0 given ex = e^x: a Taylor polynomial where the difference would cancel
+__device__ __forceinline__ float one_minus_exp(float x, float ex) {
+    float p = 1.0f + x * (1.0f / 8.0f);
+    p = 1.0f + x * (1.0f / 7.0f) * p;
+    p = 1.0f + x * (1.0f / 6.0f) * p;
+    p = 1.0f + x * (1.0f / 5.0f) * p;
+    p = 1.0f + x * (1.0f / 4.0f) * p;
+    p = 1.0f + x * (1.0f / 3.0f) * p;
+    p = 1.0f + x * (1.0f / 2.0f) * p;
+    return x > -0.35f ? -x * p : 1.0f - ex;
+}
+
+// log(1 + e^z): max(z, 0) + log(1 + e), e = e^-|z| in (0, 1]; a Taylor polynomial for small e, where 1 + e
+// would drop its digits
+__device__ __forceinline__ float softplus_fast(float z) {
+    const float e = __builtin_amdgcn_exp2f(-kLog2e * fabsf(z));
+    const float big = 0.69314718055994530942f * __builtin_amdgcn_logf(1.0f + e);
+    float p = 1.0f / 6.0f;
+    p = 1.0f / 5.0f - e * p;
+    p = 1.0f / 4.0f - e * p;
+    p = 1.0f / 3.0f - e * p;
+    p = 1.0f / 2.0f - e * p;
+    p = e * (1.0f - e * p);
+    return fmaxf(z, 0.0f) + (e < 0.0625f ? p : big);
+}
+
+template <typename T>
+__device__ __forceinline__ float softplus_as(float z) {
+    return sizeof(T) == 2 ? softplus_fast(z) : fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z)));
+}
+
 // silu of eight bf16 values, rounded to bf16
 __device__ __forceinline__ u32x4 silu8_bf16(u32x4 raw) {
     float f[8];

@@ -1,0 +1,605 @@
+// Gated delta rule with one decay per key channel: per head, with unit k, scaled unit q,
+//   S <- diag(g_t) S,   u_t = beta_t (v_t - S^T k_t),   S <- S + k_t u_t^T,   o_t = S^T q_t,
+// g = exp(-exp(A) softplus(z + dt_bias)) per key channel, beta a sigmoid, S fp32 [dp, vp].
+//
+// Chunked form (prompts, bf16), chunks of 16 tokens. With G_t the product of the decays of the chunk up to
+// token t and L_tj = product of the decays of tokens j + 1 .. t (all per channel, all <= 1):
+//   M_tj = beta_t sum_d k_td L_tjd k_jd (j < t),        P_tj = sum_d q_td L_tjd k_jd (j <= t),
+//   U = (I + M)^-1 diag(beta) (V - (G K) S),            O = (G Q) S + P U,
+//   S_new = diag(G_15) S + (L_15 K)^T U.
+//   prep   every chunk of every head at once: everything but S and V, written as MFMA operand fragments
+//          (the "image"). L cannot be split into a factor of t and one of j against the chunk's start (the
+//          second would overflow under strong decays), so pairs are grouped by the highest bit in which t
+//          and j differ: with m the middle of their common block of 2, 4, 8 or 16 tokens, L_tj is
+//          (decays m .. t)(decays j + 1 .. m - 1), both <= 1. One wave per such level, one MFMA product each.
+//   walk   chunk after chunk per head; a wave owns 16 or 32 value columns and all key channels, S in fp32
+//          accumulators. With value columns as MFMA columns throughout, every accumulator (S, V - Y, U) is
+//          the next product's operand already; images stream into LDS by direct loads, one chunk ahead.
+// 32-bit factors enter the matrix cores as two bf16 terms; a 16-deep contraction uses the two halves of a
+// 32-deep MFMA for the two terms of its left factor.
+//
+// Step kernel (decoding, and everything in float): token by token, the state in registers, one workgroup per
+// head; norm and output gate in its epilogue. For a few tokens it also convolves its inputs.
+#include "mix_conv.cuh"
+#include "mix_launchers.h"
+
+namespace astrai_mix {
+
+namespace {
+
+constexpr int kC = kDeltaChunk;
+constexpr float kUnitEps = 1e-6f;
+
+// ---- step ---------------------------------------------------------------------------------------
+constexpr int kStepThreads = 512, kStepWaves = kStepThreads / 64;
+
+// thread (rg, vq): value columns 4 vq .., state rows rg + RG i; vq runs over vqp = a power of two >= vp / 4
+template <typename T, int NR, bool FUSED>
+__global__ __launch_bounds__(kStepThreads) void delta_step_kernel(DeltaArgs a, int vqp) {
+    extern __shared__ __attribute__((aligned(16))) float sh[];
+    const int rgs = kStepThreads / vqp, rows = rgs * NR;   // rows >= dp, those past it zero
+    float* const qs = sh;                   // [rows]
+    float* const ks = qs + rows;            // [rows]
+    float* const gs = ks + rows;            // [rows]
+    float* const vs = gs + rows;            // [vp]
+    float* const red = vs + a.vp;           // [2][kStepWaves][vqp * 4]
+    float* const redk = red + 2 * kStepWaves * vqp * 4;   // [kStepWaves]
+    const int tid = threadIdx.x, lane = tid & 63;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int h = blockIdx.x, b = blockIdx.y, grp = h / (a.heads / a.kv_heads);
+    const int rg = tid / vqp, vq = tid % vqp;
+    const bool v_live = vq * 4 < a.vp;
+    const int q_col = grp * a.dp, k_col = a.kv_heads * a.dp + grp * a.dp, v_col = 2 * a.kv_heads * a.dp + h * a.vp;
+    const int64_t start = FUSED ? a.conv.positions[0] : 0;
+    float* state = a.state + ((int64_t)b * a.heads + h) * a.dp * a.vp;
+    f32x4 s[NR];
+#pragma unroll
+    for (int i = 0; i < NR; ++i) {
+        const int r = rg + rgs * i;
+        s[i] = (v_live && r < a.dp) ? *reinterpret_cast<const f32x4*>(state + (int64_t)r * a.vp + vq * 4) : f32x4{0, 0, 0, 0};
+    }
+    for (int r = a.dp + tid; r < rows; r += kStepThreads) qs[r] = ks[r] = gs[r] = 0.0f;
+    const float decay = a.decay[h];
+    for (int t = 0; t < a.seq; ++t) {
+        const int64_t row = (int64_t)b * a.seq + t;
+        auto input4 = [&](int c) -> f32x4 {
+            if constexpr (FUSED) {
+                f32x4 x = conv_at4<T>(a.conv, b, start, t, c);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) x[e] = rounded<T>(silu_as<T>(x[e]));
+                return x;
+            } else {
+                return Elem<T>::get4(static_cast<const T*>(a.qkv) + row * a.ldq + c);
+            }
+        };
+        // wave 0: q, wave 1: k (unit vectors), waves 2, 3: decays, the others: v
+        if (wave < 2) {
+            float* dst = wave ? ks : qs;
+            float sq = 0.0f;
+            for (int c = lane * 4; c < a.dp; c += 256) {
+                const f32x4 x = input4((wave ? k_col : q_col) + c);
+                sq += (x[0] * x[0] + x[1] * x[1]) + (x[2] * x[2] + x[3] * x[3]);
+                *reinterpret_cast<f32x4*>(dst + c) = x;
+            }
+            const float f = (wave ? 1.0f : a.q_scale) / sqrtf(wave_sum(sq) + kUnitEps);
+            for (int c = lane * 4; c < a.dp; c += 256) {   // (each lane what it wrote)
+                f32x4 x = *reinterpret_cast<const f32x4*>(dst + c);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) x[e] *= f;
+                *reinterpret_cast<f32x4*>(dst + c) = x;
+            }
+        } else if (wave < 4) {
+            for (int c = (wave - 2) * 64 + lane; c < a.dp; c += 128) {
+                const float z = a.z[row * a.heads * a.dp + h * a.dp + c] + a.dt_bias[h * a.dp + c];
+                const float x = -decay * softplus_as<T>(z);
+                gs[c] = sizeof(T) == 2 ? __builtin_amdgcn_exp2f(kLog2e * x) : expf(x);
+            }
+        } else {
+            for (int c = ((wave - 4) * 64 + lane) * 4; c < a.vp; c += 1024) *reinterpret_cast<f32x4*>(vs + c) = input4(v_col + c);
+        }
+        __syncthreads();
+        f32x4 pk = {0, 0, 0, 0}, pq = {0, 0, 0, 0};
+        float kq = 0.0f;
+#pragma unroll
+        for (int i = 0; i < NR; ++i) {
+            const int r = rg + rgs * i;
+            const float g = gs[r], k = ks[r], q = qs[r];
+            kq = fmaf(k, q, kq);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                s[i][e] *= g;
+                pk[e] = fmaf(s[i][e], k, pk[e]);
+                pq[e] = fmaf(s[i][e], q, pq[e]);
+            }
+        }
+        for (int off = vqp; off < kWave; off <<= 1) {
+            kq += __shfl_xor(kq, off, kWave);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                pk[e] += __shfl_xor(pk[e], off, kWave);
+                pq[e] += __shfl_xor(pq[e], off, kWave);
+            }
+        }
+        // (a wave with vqp = 64 holds one row group)
+        if (lane < vqp) {
+            *reinterpret_cast<f32x4*>(red + (wave * vqp + vq) * 4) = pk;
+            *reinterpret_cast<f32x4*>(red + ((kStepWaves + wave) * vqp + vq) * 4) = pq;
+        }
+        if (lane == 0) redk[wave] = kq;
+        __syncthreads();
+        f32x4 o = {0, 0, 0, 0}, u = {0, 0, 0, 0};
+        kq = 0.0f;
+#pragma unroll
+        for (int w = 0; w < kStepWaves; ++w) {
+            u += *reinterpret_cast<const f32x4*>(red + (w * vqp + vq) * 4);
+            o += *reinterpret_cast<const f32x4*>(red + ((kStepWaves + w) * vqp + vq) * 4);
+            kq += redk[w];
+        }
+        const float beta = sigmoid(Elem<T>::get(static_cast<const T*>(a.proj) + row * a.ld + a.b_off + h));
+        const f32x4 v = v_live ? *reinterpret_cast<const f32x4*>(vs + vq * 4) : f32x4{0, 0, 0, 0};
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            u[e] = beta * (v[e] - u[e]);
+            o[e] = fmaf(u[e], kq, o[e]);
+        }
+#pragma unroll
+        for (int i = 0; i < NR; ++i) {
+            const float k = ks[rg + rgs * i];
+#pragma unroll
+            for (int e = 0; e < 4; ++e) s[i][e] = fmaf(k, u[e], s[i][e]);
+        }
+        if (rg == 0) {   // the first vqp lanes of wave 0
+            float sq = v_live ? (o[0] * o[0] + o[1] * o[1]) + (o[2] * o[2] + o[3] * o[3]) : 0.0f;
+            for (int off = vqp / 2; off; off >>= 1) sq += __shfl_xor(sq, off, kWave);
+            if (v_live) {
+                const float f = 1.0f / sqrtf(sq / (float)a.vdim + a.eps);
+                const int c = h * a.vp + vq * 4;
+                const f32x4 z = Elem<T>::get4(static_cast<const T*>(a.gate) + row * a.ldg + c);
+                const f32x4 w = *reinterpret_cast<const f32x4*>(a.norm_w + vq * 4);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) o[e] = o[e] * f * w[e] * sigmoid(z[e]);
+                Elem<T>::put4(static_cast<T*>(a.out) + row * a.heads * a.vp + c, o);
+            }
+        }
+        __syncthreads();   // vectors and partial sums of this token are no longer read
+    }
+#pragma unroll
+    for (int i = 0; i < NR; ++i) {
+        const int r = rg + rgs * i;
+        if (v_live && r < a.dp) *reinterpret_cast<f32x4*>(state + (int64_t)r * a.vp + vq * 4) = s[i];
+    }
+    if constexpr (FUSED) {
+        // the last inputs into the ring, rows that no workgroup of this launch reads; a group's first head
+        // writes the shared q and k
+        const bool first = h % (a.heads / a.kv_heads) == 0;
+        const int n = (first ? 2 * a.dp : 0) + a.vp;
+        for (int c = tid * 4; c < n; c += kStepThreads * 4) {
+            const int d = first ? c : c + 2 * a.dp;
+            const int col = d < a.dp ? q_col + d : d < 2 * a.dp ? k_col + d - a.dp : v_col + d - 2 * a.dp;
+            for (int t = max(a.seq - a.conv.taps + 1, 0); t < a.seq; ++t) ring_put4<T>(a.conv, b, start, t, col);
+        }
+    }
+}
+
+// ---- chunk: image of a (sequence, head, chunk), in fragments of 64 lanes x 16 bytes ---------------------
+//   [0, NS)       G K, high terms: lane (g, c16), step s: row c16, channels 32 s + 4 g .. and 32 s + 16 + 4 g ..
+//   [NS, 2 NS)    its low terms
+//   [2 NS, 4 NS)  G Q likewise
+//   [4 NS, 6 NS)  (L_15 K)^T: tile i: row = channel 16 i + c16, tokens 4 g .., high terms then low
+//   6 NS          (I + M)^-1 diag(beta): row c16, tokens 4 g .., high terms then low
+//   6 NS + 1      P likewise
+//   then dp floats: G_15
+template <int DP>
+struct Image {
+    static constexpr int NS = DP / 32;
+    static constexpr int kFrags = 6 * NS + 2;
+    static constexpr int kBytes = kFrags * 1024 + DP * 4;
+    static constexpr int kDma = (kBytes + 1023) / 1024;    // 1 KiB pieces; memory per image is whole pieces
+};
+
+__device__ __forceinline__ u32x4 split4(f32x4 v) {   // four high terms, four low terms
+    uint32_t h0, l0, h1, l1;
+    split2(v[0], v[1], h0, l0);
+    split2(v[2], v[3], h1, l1);
+    return u32x4{h0, h1, l0, l1};
+}
+
+__device__ __forceinline__ void put_split(uint8_t* hi, uint8_t* lo, int off, float v) {
+    uint32_t h, l;
+    split2(v, 0.0f, h, l);
+    *reinterpret_cast<uint16_t*>(hi + off) = (uint16_t)h;
+    *reinterpret_cast<uint16_t*>(lo + off) = (uint16_t)l;
+}
+
+template <int DP>
+__global__ __launch_bounds__(256) void delta_prep_kernel(DeltaArgs a, int chunks) {
+    constexpr int NS = DP / 32, kRow = DP * 2 + 16, kMat = kC * kRow;   // bytes
+    constexpr int kPer = (DP + 127) / 128;        // channels per thread
+    extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
+    uint8_t* const mats = lds;                    // [4 levels][k hi, k lo, q hi, q lo][kC][kRow]
+    float* const lg = reinterpret_cast<float*>(lds + 16 * kMat);   // [kC][DP] decays
+    float* const inv = lg + kC * DP;              // [2][kC]: factor of q, of k
+    float* const diag = inv + 2 * kC;             // [kC]
+    float* const beta = diag + kC;                // [kC]
+    float* const ms = beta + kC;                  // [kC][20]
+    float* const ps = ms + kC * 20;               // [kC][20]
+    const int tid = threadIdx.x, lane = tid & 63, c16 = lane & 15, g = lane >> 4;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int chunk = blockIdx.x, h = blockIdx.y, b = blockIdx.z, grp = h / (a.heads / a.kv_heads);
+    const int t0 = chunk * kC, n = min(kC, a.seq - t0);
+    const int64_t row0 = (int64_t)b * a.seq + t0;
+    const uint16_t* q = static_cast<const uint16_t*>(a.qkv) + row0 * a.ldq + grp * a.dp;
+    const uint16_t* k = q + a.kv_heads * a.dp;
+    uint8_t* image = static_cast<uint8_t*>(a.image) + (((int64_t)b * a.heads + h) * chunks + chunk) * (Image<DP>::kDma * 1024);
+
+    // norms: 16 lanes per token, which also give q . k of the same token
+    {
+        const int t = tid >> 4, l = tid & 15;
+        float sq = 0.0f, sk = 0.0f, qk = 0.0f;
+        if (t < n)
+            for (int c = l * 8; c < a.dp; c += 128) {
+                float x[8], y[8];
+                w8a8::unpack8(*reinterpret_cast<const u32x4*>(q + (int64_t)t * a.ldq + c), x);
+                w8a8::unpack8(*reinterpret_cast<const u32x4*>(k + (int64_t)t * a.ldq + c), y);
+#pragma unroll
+                for (int e = 0; e < 8; ++e) {
+                    sq = fmaf(x[e], x[e], sq);
+                    sk = fmaf(y[e], y[e], sk);
+                    qk = fmaf(x[e], y[e], qk);
+                }
+            }
+#pragma unroll
+        for (int off = 8; off; off >>= 1) {
+            sq += __shfl_xor(sq, off, kWave);
+            sk += __shfl_xor(sk, off, kWave);
+            qk += __shfl_xor(qk, off, kWave);
+        }
+        if (l == 0) {
+            const float fq = a.q_scale / sqrtf(sq + kUnitEps), fk = 1.0f / sqrtf(sk + kUnitEps);
+            inv[t] = fq;
+            inv[kC + t] = fk;
+            diag[t] = qk * fq * fk;
+            beta[t] = t < n ? sigmoid(Elem<uint16_t>::get(static_cast<const uint16_t*>(a.proj) + (row0 + t) * a.ld + a.b_off + h))
+                            : 0.0f;
+        }
+    }
+    // decays: each half of the workgroup eight tokens
+    {
+        const float decay = a.decay[h];
+        const int half = tid >> 7;
+        for (int d = tid & 127; d < DP; d += 128) {
+            const float bias = d < a.dp ? a.dt_bias[h * a.dp + d] : 0.0f;
+#pragma unroll
+            for (int i = 0; i < 8; ++i) {
+                const int t = half * 8 + i;
+                float x = 1.0f;
+                if (t < n && d < a.dp)
+                    x = __builtin_amdgcn_exp2f(-kLog2e * decay * softplus_fast(a.z[(row0 + t) * a.heads * a.dp + h * a.dp + d] + bias));
+                lg[t * DP + d] = x;
+            }
+        }
+    }
+    __syncthreads();
+    // operands: half 0 the keys, half 1 the queries, a channel per thread
+    {
+        const bool is_q = tid >= 128;
+        const uint16_t* src = is_q ? q : k;
+        const float* f = inv + (is_q ? 0 : kC);
+#pragma unroll
+        for (int p = 0; p < kPer; ++p) {
+            const int d = (tid & 127) + p * 128;
+            if (d < DP) {
+                float x[kC], dec[kC];
+#pragma unroll
+                for (int t = 0; t < kC; ++t) {
+                    x[t] = (t < n && d < a.dp) ? Elem<uint16_t>::get(src + (int64_t)t * a.ldq + d) * f[t] : 0.0f;
+                    dec[t] = lg[t * DP + d];
+                }
+                // levels: blocks of 2 hb tokens, middle m; upper tokens take decays m .. t, lower ones j + 1 .. m - 1
+#pragma unroll
+                for (int lv = 0; lv < 4; ++lv) {
+                    constexpr int kHalf[4] = {8, 4, 2, 1};
+                    const int hb = kHalf[lv];
+                    uint8_t* hi = mats + (lv * 4 + (is_q ? 2 : 0)) * kMat;
+                    uint8_t* lo = hi + kMat;
+#pragma unroll
+                    for (int m = hb; m < kC; m += 2 * hb) {
+                        float w = 1.0f;
+#pragma unroll
+                        for (int t = m; t < m + hb; ++t) {
+                            w *= dec[t];
+                            put_split(hi, lo, t * kRow + d * 2, x[t] * w);
+                        }
+                        if (!is_q) {
+                            w = 1.0f;
+#pragma unroll
+                            for (int j = m - 1; j >= m - hb; --j) {
+                                put_split(hi, lo, j * kRow + d * 2, x[j] * w);
+                                w *= dec[j];
+                            }
+                        }
+                    }
+                }
+                // G K, G Q: into the image, channels in the order of the accumulators' rows
+                {
+                    const int s = d >> 5, r = d & 31, pos = ((r & 15) >> 2) * 8 + (r >> 4) * 4 + (r & 3);   // 8 gg + j
+                    uint8_t* hi = image + ((is_q ? 2 * NS : 0) + s) * 1024 + (pos >> 3) * 256 + (pos & 7) * 2;
+                    uint8_t* lo = hi + NS * 1024;
+                    float w = 1.0f;
+#pragma unroll
+                    for (int t = 0; t < kC; ++t) {
+                        w *= dec[t];
+                        put_split(hi, lo, t * 16, x[t] * w);
+                    }
+                    if (!is_q) reinterpret_cast<float*>(image + Image<DP>::kFrags * 1024)[d] = w;
+                }
+                if (!is_q) {
+                    float w = 1.0f;
+#pragma unroll
+                    for (int j = kC - 1; j >= 0; --j) {
+                        x[j] *= w;
+                        w *= dec[j];
+                    }
+                    uint8_t* dst = image + (4 * NS + (d >> 4)) * 1024 + (d & 15) * 16;
+#pragma unroll
+                    for (int gg = 0; gg < 4; ++gg)
+                        *reinterpret_cast<u32x4*>(dst + gg * 256) = split4(f32x4{x[4 * gg], x[4 * gg + 1], x[4 * gg + 2], x[4 * gg + 3]});
+                }
+            }
+        }
+    }
+    __syncthreads();
+    // pairs: a wave per level; the level of (t, j) is the highest bit of t ^ j
+    {
+        const int hb = 8 >> wave;
+        const uint8_t* base = mats + wave * 4 * kMat + c16 * kRow + 16 * g;
+        f32x4 dm = {0, 0, 0, 0}, dq = {0, 0, 0, 0};
+#pragma unroll
+        for (int s = 0; s < NS; ++s) {
+            const u32x4 kh = *reinterpret_cast<const u32x4*>(base + s * 64);
+            const u32x4 kl = *reinterpret_cast<const u32x4*>(base + kMat + s * 64);
+            const u32x4 qh = *reinterpret_cast<const u32x4*>(base + 2 * kMat + s * 64);
+            const u32x4 ql = *reinterpret_cast<const u32x4*>(base + 3 * kMat + s * 64);
+            dm = mfma16(kh, kh, dm);
+            dm = mfma16(kh, kl, dm);
+            dm = mfma16(kl, kh, dm);
+            dq = mfma16(qh, kh, dq);
+            dq = mfma16(qh, kl, dq);
+            dq = mfma16(ql, kh, dq);
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const int t = 4 * g + e, j = c16, x = t ^ j;
+            if (t > j && x >= hb && x < 2 * hb) {
+                ms[t * 20 + j] = beta[t] * dm[e];
+                ps[t * 20 + j] = dq[e];
+            } else if (wave == 0 && t <= j) {
+                ms[t * 20 + j] = 0.0f;
+                ps[t * 20 + j] = t == j ? diag[t] : 0.0f;
+            }
+        }
+    }
+    __syncthreads();
+    if (wave == 0) {
+        // row c16 of X = (I + M)^-1 from X (I + M) = I, last column first
+        float x[kC];
+#pragma unroll
+        for (int j = 0; j < kC; ++j) x[j] = j == c16 ? 1.0f : 0.0f;
+#pragma unroll
+        for (int s = kC - 1; s >= 1; --s) {
+            float m[kC];
+#pragma unroll
+            for (int j = 0; j < s; j += 4) {
+                const f32x4 v = *reinterpret_cast<const f32x4*>(ms + s * 20 + j);
+                m[j] = v[0];
+                m[j + 1] = v[1];
+                m[j + 2] = v[2];
+                m[j + 3] = v[3];
+            }
+#pragma unroll
+            for (int j = 0; j < s; ++j) x[j] = fmaf(-x[s], m[j], x[j]);
+        }
+        f32x4 mine = {0, 0, 0, 0};
+#pragma unroll
+        for (int gg = 0; gg < 4; ++gg)
+            if (g == gg) mine = f32x4{x[4 * gg], x[4 * gg + 1], x[4 * gg + 2], x[4 * gg + 3]};
+#pragma unroll
+        for (int e = 0; e < 4; ++e) mine[e] *= beta[4 * g + e];
+        *reinterpret_cast<u32x4*>(image + 6 * NS * 1024 + lane * 16) = split4(mine);
+    } else if (wave == 1) {
+        *reinterpret_cast<u32x4*>(image + (6 * NS + 1) * 1024 + lane * 16) =
+            split4(*reinterpret_cast<const f32x4*>(ps + c16 * 20 + 4 * g));
+    }
+}
+
+__device__ __forceinline__ void lds_dma16(__amdgpu_buffer_rsrc_t r, uint8_t* lds_wave_base, uint32_t voff) {
+    __builtin_amdgcn_raw_ptr_buffer_load_lds(r, (__attribute__((address_space(3))) void*)lds_wave_base, 16, voff, 0, 0, 0);
+}
+
+// VT: 16-column value tiles per wave
+template <int DP, int VT>
+__global__ __launch_bounds__(256, DP <= 128 ? 2 : 1) void delta_walk_kernel(DeltaArgs a, int chunks) {
+    constexpr int NS = DP / 32, NT = DP / 16, kBuf = Image<DP>::kDma * 1024;
+    extern __shared__ __attribute__((aligned(1024))) uint8_t lds[];   // two images
+    const int tid = threadIdx.x, lane = tid & 63, c16 = lane & 15, g = lane >> 4;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int h = blockIdx.y, b = blockIdx.z;
+    const int v0 = ((int)blockIdx.x * 4 + wave) * (16 * VT);
+    const uint8_t* images = static_cast<const uint8_t*>(a.image) + ((int64_t)b * a.heads + h) * chunks * kBuf;
+    auto dma = [&](int c) {
+        const __amdgpu_buffer_rsrc_t r = w8a8::make_rsrc(images + (int64_t)c * kBuf, c < chunks ? kBuf : 0);
+        uint8_t* dst = lds + (c & 1) * kBuf;
+        for (int i = wave; i < Image<DP>::kDma; i += 4) lds_dma16(r, dst + i * 1024, i * 1024 + lane * 16);
+    };
+    const uint16_t* vsrc = static_cast<const uint16_t*>(a.qkv) + (int64_t)b * a.seq * a.ldq + 2 * a.kv_heads * a.dp + h * a.vp;
+    float* state = a.state + ((int64_t)b * a.heads + h) * a.dp * a.vp;
+    // S: rows 16 i + 4 g + e, columns v0 + 16 vt + c16
+    f32x4 st[NT][VT];
+#pragma unroll
+    for (int i = 0; i < NT; ++i)
+#pragma unroll
+        for (int vt = 0; vt < VT; ++vt)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const int d = 16 * i + 4 * g + e, v = v0 + 16 * vt + c16;
+                st[i][vt][e] = (d < a.dp && v < a.vp) ? state[(int64_t)d * a.vp + v] : 0.0f;
+            }
+    uint16_t vr[VT][4];
+    auto fetch_v = [&](int c) {
+#pragma unroll
+        for (int vt = 0; vt < VT; ++vt)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const int t = c * kC + 4 * g + e, v = v0 + 16 * vt + c16;
+                vr[vt][e] = (t < a.seq && v < a.vp) ? vsrc[(int64_t)t * a.ldq + v] : 0;
+            }
+    };
+    dma(0);
+    fetch_v(0);
+    for (int c = 0; c < chunks; ++c) {
+        __builtin_amdgcn_s_waitcnt(0x0070);   // vmcnt(0) lgkmcnt(0)
+        __syncthreads();                      // image c is there, image c - 1 is no longer read
+        dma(c + 1);
+        f32x4 x[VT];
+#pragma unroll
+        for (int vt = 0; vt < VT; ++vt)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) x[vt][e] = w8a8::bf16_to_f32(vr[vt][e]);
+        fetch_v(c + 1);
+        const uint8_t* im = lds + (c & 1) * kBuf;
+        auto frag = [&](int i) { return *reinterpret_cast<const u32x4*>(im + i * 1024 + lane * 16); };
+        f32x4 y[VT], o[VT];
+#pragma unroll
+        for (int vt = 0; vt < VT; ++vt) y[vt] = o[vt] = f32x4{0, 0, 0, 0};
+#pragma unroll
+        for (int s = 0; s < NS; ++s) {
+            const u32x4 kh = frag(s), kl = frag(NS + s), qh = frag(2 * NS + s), ql = frag(3 * NS + s);
+#pragma unroll
+            for (int vt = 0; vt < VT; ++vt) {
+                const u32x4 p0 = split4(st[2 * s][vt]), p1 = split4(st[2 * s + 1][vt]);
+                const u32x4 sh = {p0[0], p0[1], p1[0], p1[1]}, sl = {p0[2], p0[3], p1[2], p1[3]};
+                y[vt] = mfma16(kh, sh, y[vt]);
+                o[vt] = mfma16(qh, sh, o[vt]);
+                y[vt] = mfma16(kl, sh, y[vt]);
+                o[vt] = mfma16(ql, sh, o[vt]);
+                y[vt] = mfma16(kh, sl, y[vt]);
+                o[vt] = mfma16(qh, sl, o[vt]);
+            }
+        }
+        const u32x4 tf = frag(6 * NS), pf = frag(6 * NS + 1);
+        u32x4 uh[VT], ul[VT];
+#pragma unroll
+        for (int vt = 0; vt < VT; ++vt) {
+            const u32x4 p = split4(x[vt] - y[vt]);
+            f32x4 u = {0, 0, 0, 0};
+            u = mfma16(tf, u32x4{p[0], p[1], p[0], p[1]}, u);
+            u = mfma16(tf, u32x4{p[2], p[3], p[2], p[3]}, u);
+            const u32x4 w = split4(u);
+            uh[vt] = u32x4{w[0], w[1], w[0], w[1]};
+            ul[vt] = u32x4{w[2], w[3], w[2], w[3]};
+            o[vt] = mfma16(pf, uh[vt], o[vt]);
+            o[vt] = mfma16(pf, ul[vt], o[vt]);
+        }
+        const float* gam = reinterpret_cast<const float*>(im + Image<DP>::kFrags * 1024) + 4 * g;
+#pragma unroll
+        for (int i = 0; i < NT; ++i) {
+            const f32x4 gg = *reinterpret_cast<const f32x4*>(gam + 16 * i);
+            const u32x4 kf = frag(4 * NS + i);
+#pragma unroll
+            for (int vt = 0; vt < VT; ++vt) {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) st[i][vt][e] *= gg[e];
+                st[i][vt] = mfma16(kf, uh[vt], st[i][vt]);
+                st[i][vt] = mfma16(kf, ul[vt], st[i][vt]);
+            }
+        }
+#pragma unroll
+        for (int vt = 0; vt < VT; ++vt)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const int t = c * kC + 4 * g + e, v = v0 + 16 * vt + c16;
+                if (t < a.seq && v < a.vp)
+                    Elem<uint16_t>::put(static_cast<uint16_t*>(a.out) + (((int64_t)b * a.seq + t) * a.heads + h) * a.vp + v, o[vt][e]);
+            }
+    }
+#pragma unroll
+    for (int i = 0; i < NT; ++i)
+#pragma unroll
+        for (int vt = 0; vt < VT; ++vt)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const int d = 16 * i + 4 * g + e, v = v0 + 16 * vt + c16;
+                if (d < a.dp && v < a.vp) state[(int64_t)d * a.vp + v] = st[i][vt][e];
+            }
+}
+
+template <int DP, int VT>
+void walk_t(const DeltaArgs& a, int chunks, hipStream_t stream) {
+    constexpr int shared = 2 * Image<DP>::kDma * 1024;
+    static const hipError_t once = hipFuncSetAttribute(reinterpret_cast<const void*>(&delta_walk_kernel<DP, VT>),
+                                                       hipFuncAttributeMaxDynamicSharedMemorySize, shared);
+    (void)once;
+    const dim3 grid((unsigned)((a.vp + 64 * VT - 1) / (64 * VT)), (unsigned)a.heads, (unsigned)a.batch);
+    delta_walk_kernel<DP, VT><<<grid, 256, shared, stream>>>(a, chunks);
+}
+
+template <int DP>
+void chunk_t(const DeltaArgs& a, hipStream_t stream) {
+    constexpr int shared = 16 * kC * (DP * 2 + 16) + kC * DP * 4 + 4 * kC * 4 + 2 * kC * 20 * 4;
+    static const hipError_t once = hipFuncSetAttribute(reinterpret_cast<const void*>(&delta_prep_kernel<DP>),
+                                                       hipFuncAttributeMaxDynamicSharedMemorySize, shared);
+    (void)once;
+    const int chunks = (a.seq + kC - 1) / kC;
+    delta_prep_kernel<DP><<<dim3((unsigned)chunks, (unsigned)a.heads, (unsigned)a.batch), 256, shared, stream>>>(a, chunks);
+    // wide slices read every image once; narrow ones make more workgroups
+    if (DP <= 128 && a.vp > 64 && (int64_t)a.batch * a.heads >= 256) walk_t<DP, 2>(a, chunks, stream);
+    else walk_t<DP, 1>(a, chunks, stream);
+}
+
+template <typename T, int NR>
+void step_n(const DeltaArgs& a, bool fused, int vqp, hipStream_t stream) {
+    const int shared = (3 * (kStepThreads / vqp) * NR + a.vp + 2 * kStepWaves * vqp * 4 + kStepWaves) * (int)sizeof(float);
+    const dim3 grid((unsigned)a.heads, (unsigned)a.batch);
+    if (fused) delta_step_kernel<T, NR, true><<<grid, kStepThreads, shared, stream>>>(a, vqp);
+    else delta_step_kernel<T, NR, false><<<grid, kStepThreads, shared, stream>>>(a, vqp);
+}
+
+int step_vqp(int vp) {
+    int vqp = 8;
+    while (vqp * 4 < vp) vqp *= 2;
+    return vqp;
+}
+
+template <typename T>
+void step_t(const DeltaArgs& a, bool fused, hipStream_t stream) {
+    const int vqp = step_vqp(a.vp), rows = (a.dp * vqp + kStepThreads - 1) / kStepThreads;
+    if (rows <= 4) step_n<T, 4>(a, fused, vqp, stream);
+    else if (rows <= 8) step_n<T, 8>(a, fused, vqp, stream);
+    else if (rows <= 16) step_n<T, 16>(a, fused, vqp, stream);
+    else step_n<T, 32>(a, fused, vqp, stream);
+}
+
+}  // namespace
+
+bool delta_step_supported(int dp, int vp) { return vp <= 256 && dp <= 1024 && dp * step_vqp(vp) <= 32 * kStepThreads; }
+
+void launch_delta_step(const DeltaArgs& a, bool fused, int dtype, hipStream_t stream) {
+    if (dtype) step_t<float>(a, fused, stream);
+    else step_t<uint16_t>(a, fused, stream);
+}
+
+bool delta_chunk_supported(int dp, int vp) { return dp <= 256 && vp > 0; }
+
+int64_t delta_image_bytes(int dp) {
+    const int kb = dp <= 32 ? Image<32>::kDma : dp <= 64 ? Image<64>::kDma : dp <= 128 ? Image<128>::kDma : Image<256>::kDma;
+    return (int64_t)kb * 1024;
+}
+
+void launch_delta_chunk(const DeltaArgs& a, hipStream_t stream) {
+    if (a.dp <= 32) chunk_t<32>(a, stream);
+    else if (a.dp <= 64) chunk_t<64>(a, stream);
+    else if (a.dp <= 128) chunk_t<128>(a, stream);
+    else chunk_t<256>(a, stream);
+}
+
+}  // namespace astrai_mix

@@ -1,6 +1,10 @@
-// Causal sliding-window attention of a block of new tokens (prompt, whole or in portions) for
-// heads with their own keys and values plus one rotated key part shared by all heads: bf16
-// MFMAs, fp32 scores, weights and sums, per-head output gate in the epilogue.
+// Causal sliding-window attention of a block of new tokens (prompt, whole or in portions): bf16
+// MFMAs, fp32 scores, weights and sums, output gate in the epilogue. Two kinds of heads:
+//   latent        each head has its own keys and values, plus one rotated key part shared by all
+//                 heads; a gate per head
+//   grouped-query (GQA) `group` heads share keys and values; soft-capped scores, a sink (one more term
+//                 exp(0) in the softmax denominator: the running maximum starts at 0 and the sum at
+//                 1), a gate per element, each optional
 //
 // One workgroup per (sequence, head, 128 query tokens), wave r taking 32 of them; key tiles of 32,
 // only those some query of the wave can see:
@@ -43,8 +47,8 @@ __device__ __forceinline__ int row_swizzle(int row) {
     return (row / R) & (C >= 16 ? 15 : C - 1);
 }
 
-template <int DN, int DR, int DV>
-__global__ __launch_bounds__(256, 2) void latent_prefill_kernel(LatentPrefillArgs a, LatentDims d) {
+template <int DN, int DR, int DV, bool GQA>
+__global__ __launch_bounds__(256, 2) void mix_prefill_kernel(LatentPrefillArgs a, LatentDims d) {
     constexpr int NKN = DN / 16, NKR = DR / 16, NK = NKN + NKR;   // score MFMA steps
     constexpr int NV = DV / 32;                                   // value column tiles
     constexpr int CN = DN / 8, CR = DR / 8, CV = DV / 8;          // 16-byte chunks per row
@@ -61,6 +65,7 @@ __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(LatentPrefillArg
     const int nqb = (a.seq + kQB - 1) / kQB;
     const int qb = nqb - 1 - (int)(blockIdx.x / groups), bh = (int)(blockIdx.x % groups);   // longest key ranges first
     const int b = bh / d.heads, head = bh % d.heads;
+    const int kv_head = GQA ? head / a.group : head, kv_heads = GQA ? d.heads / a.group : d.heads;
     const int dk = d.dn + d.dr;
     const int q0 = qb * kQB;
 
@@ -87,21 +92,23 @@ __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(LatentPrefillArg
         }
     }
 
-    const int64_t ldkv = (int64_t)d.heads * (d.dn + d.vp) * 2, ldc = (d.rp + d.dr) * 2;   // bytes
+    const int64_t ldkv = (int64_t)kv_heads * (d.dn + d.vp) * 2, ldc = (d.rp + d.dr) * 2;   // bytes
     const uint8_t* kv = static_cast<const uint8_t*>(a.kv) + ((int64_t)b * a.n_keys - a.key_base) * ldkv +
-                        (int64_t)head * (d.dn + d.vp) * 2;
+                        (int64_t)kv_head * (d.dn + d.vp) * 2;
     const uint8_t* kr = static_cast<const uint8_t*>(a.cache) + (int64_t)b * a.max_len * ldc + d.rp * 2;
     // per-lane offsets from a block's first row; a chunk past the real columns asks for nothing
-    uint32_t on[JN], orr[JR], ov[JV];
+    uint32_t on[JN], orr[DR ? JR : 1], ov[JV];
 #pragma unroll
     for (int j = 0; j < JN; ++j) {
         const int row = (wave * JN + j) * (64 / CN) + lane / CN, c = (lane % CN) ^ row_swizzle<CN>(row & 31);
         on[j] = c * 8 < d.dn ? (uint32_t)(row * ldkv) + c * 16 : w8a8::kOutOfRange;
     }
+    if constexpr (DR > 0) {
 #pragma unroll
-    for (int j = 0; j < JR; ++j) {
-        const int row = (wave * JR + j) * (64 / CR) + lane / CR, c = (lane % CR) ^ row_swizzle<CR>(row & 31);
-        orr[j] = c * 8 < d.dr ? (uint32_t)(row * ldc) + c * 16 : w8a8::kOutOfRange;
+        for (int j = 0; j < JR; ++j) {
+            const int row = (wave * JR + j) * (64 / CR) + lane / CR, c = (lane % CR) ^ row_swizzle<CR>(row & 31);
+            orr[j] = c * 8 < d.dr ? (uint32_t)(row * ldc) + c * 16 : w8a8::kOutOfRange;
+        }
     }
     // values: chunk bit 2 (and 3) by the row inside its group of four
     auto v_swizzle = [](int row) { return CV == 16 ? 4 * (row & 3) : 4 * ((row >> 1) & 1); };
@@ -118,16 +125,18 @@ __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(LatentPrefillArg
     auto dma_k = [&](int t0) {
         const int key = kmin + t0 * 32, rows = min(kmax - key + 1, kKB);
         const __amdgpu_buffer_rsrc_t rn = rows_rsrc(kv + (int64_t)key * ldkv, rows, ldkv, d.dn * 2);
-        const __amdgpu_buffer_rsrc_t rr = rows_rsrc(kr + (int64_t)key * ldc, rows, ldc, d.dr * 2);
 #pragma unroll
         for (int j = 0; j < JN; ++j) {
             const int inst = wave * JN + j;
             lds_dma16(rn, lds + ((t0 + inst / IN) & 3) * kTile + (inst % IN) * 1024, on[j]);
         }
+        if constexpr (DR > 0) {
+            const __amdgpu_buffer_rsrc_t rr = rows_rsrc(kr + (int64_t)key * ldc, rows, ldc, d.dr * 2);
 #pragma unroll
-        for (int j = 0; j < JR; ++j) {
-            const int inst = wave * JR + j;
-            lds_dma16(rr, lds + ((t0 + inst / IR) & 3) * kTile + 32 * kNRow + (inst % IR) * 1024, orr[j]);
+            for (int j = 0; j < JR; ++j) {
+                const int inst = wave * JR + j;
+                lds_dma16(rr, lds + ((t0 + inst / IR) & 3) * kTile + 32 * kNRow + (inst % IR) * 1024, orr[j]);
+            }
         }
     };
     auto dma_v = [&](int kb) {
@@ -146,16 +155,20 @@ __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(LatentPrefillArg
     // maximum once some query has outgrown it by 2^kSlack (until then weights reach 2^kSlack). It
     // starts far below any score and far above a hidden key's.
     constexpr float kSlack = 8.0f;
-    float m_run = 1e-5f * kNegBig, l_run = 0.0f;
-    const float c = d.scale * kLog2e;
+    const bool sink = GQA && a.sink;
+    float m_run = sink ? 0.0f : 1e-5f * kNegBig, l_run = sink && h2 == 0 ? 1.0f : 0.0f;
+    // capped scores leave mask_max4 in log2 units
+    const bool capped = GQA && a.softcap > 0.0f;
+    const float c = capped ? 1.0f : d.scale * kLog2e;
+    const float cap_in = capped ? d.scale / a.softcap : 0.0f, cap_out = a.softcap * kLog2e;
     const f32x16 zero16 = {0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f,
                            0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f};
     // key operand of step ks: chunk (2 ks + h2) ^ swizzle of this lane's row. Rows are powers of two and
     // tiles whole rows, so the step XORs into the whole byte offset: one address register per tile.
     const int kn_lane = qi * kNRow + ((h2 ^ row_swizzle<CN>(qi)) << 4);
-    const int kr_lane = 32 * kNRow + qi * kRRow + ((h2 ^ row_swizzle<CR>(qi)) << 4);
+    const int kr_lane = 32 * kNRow + qi * kRRow + ((h2 ^ row_swizzle<DR ? CR : CN>(qi)) << 4);
     auto k_frag = [&](int slot, int ks) -> u32x4 {
-        const int off = ks < NKN ? ((slot + kn_lane) ^ (ks << 5)) : ((slot + kr_lane) ^ ((ks - NKN) << 5));
+        const int off = (DR == 0 || ks < NKN) ? ((slot + kn_lane) ^ (ks << 5)) : ((slot + kr_lane) ^ ((ks - NKN) << 5));
         return *reinterpret_cast<const u32x4*>(lds + off);
     };
     // V^T operand of 32 columns x 16 keys: lane half takes rows 4 h2 .. and 8 + 4 h2 .. of the step
@@ -171,6 +184,7 @@ __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(LatentPrefillArg
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
             const int e = 4 * g + j, key = kmin + T * 32 + g * 8 + h2 * 4 + j;
+            if (capped) s[e] = cap_out * tanh_fast(s[e] * cap_in);
             s[e] = (key <= pq && key >= plo) ? s[e] : kNegBig;
             m = fmaxf(m, s[e]);
         }
@@ -255,15 +269,26 @@ __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(LatentPrefillArg
     if (!w_live) return;
     // normalise, gate, and write through LDS (idle by now), so that rows leave in whole pieces
     const float l = l_run + __shfl_xor(l_run, 32, kWave);
-    const float f = sigmoid(Elem<uint16_t>::get(static_cast<const uint16_t*>(a.proj) + tok * a.ld + a.g_off + head)) / l;
+    const uint16_t* gate = static_cast<const uint16_t*>(a.proj) + tok * a.ld + a.g_off;
+    float f = 1.0f / l;
+    if constexpr (GQA) gate += head * d.vp;
+    else f *= sigmoid(Elem<uint16_t>::get(gate + head));
     uint8_t* const mine = lds + wave * 32 * kVRow;
 #pragma unroll
     for (int i = 0; i < NV; ++i)
 #pragma unroll
         for (int g = 0; g < 4; ++g) {
             const int chunk = (4 * i + g) ^ (qi & (CV - 1));
-            Elem<uint16_t>::put4(reinterpret_cast<uint16_t*>(mine + qi * kVRow + chunk * 16 + h2 * 8),
-                                 f32x4{o[i][4 * g] * f, o[i][4 * g + 1] * f, o[i][4 * g + 2] * f, o[i][4 * g + 3] * f});
+            f32x4 v = {o[i][4 * g] * f, o[i][4 * g + 1] * f, o[i][4 * g + 2] * f, o[i][4 * g + 3] * f};
+            if constexpr (GQA) {
+                const int col = 32 * i + 8 * g + 4 * h2;
+                if (a.g_off >= 0 && col < d.vp) {
+                    const f32x4 z = Elem<uint16_t>::get4(gate + col);
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) v[e] *= sigmoid_fast(z[e]);
+                }
+            }
+            Elem<uint16_t>::put4(reinterpret_cast<uint16_t*>(mine + qi * kVRow + chunk * 16 + h2 * 8), v);
         }
     uint16_t* const out = static_cast<uint16_t*>(a.out) + (((int64_t)b * a.seq + q0 + wave * 32) * d.heads + head) * d.vp;
 #pragma unroll
@@ -275,26 +300,26 @@ __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(LatentPrefillArg
     }
 }
 
-template <int DN, int DR, int DV>
+template <int DN, int DR, int DV, bool GQA>
 void prefill_t(const LatentPrefillArgs& a, const LatentDims& d, hipStream_t stream) {
     constexpr int shared = 4 * 32 * (DN + DR) * 2 + 2 * kKB * DV * 2;
-    static const hipError_t once = hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_prefill_kernel<DN, DR, DV>),
+    static const hipError_t once = hipFuncSetAttribute(reinterpret_cast<const void*>(&mix_prefill_kernel<DN, DR, DV, GQA>),
                                                        hipFuncAttributeMaxDynamicSharedMemorySize, shared);
     (void)once;
     const unsigned blocks = (unsigned)(((a.seq + kQB - 1) / kQB) * a.batch * d.heads);
-    latent_prefill_kernel<DN, DR, DV><<<blocks, 256, shared, stream>>>(a, d);
+    mix_prefill_kernel<DN, DR, DV, GQA><<<blocks, 256, shared, stream>>>(a, d);
 }
 
-template <int DN, int DR>
+template <int DN, int DR, bool GQA>
 void prefill_v(const LatentPrefillArgs& a, const LatentDims& d, hipStream_t stream) {
-    if (d.vp <= 64) prefill_t<DN, DR, 64>(a, d, stream);
-    else prefill_t<DN, DR, 128>(a, d, stream);
+    if (d.vp <= 64) prefill_t<DN, DR, 64, GQA>(a, d, stream);
+    else prefill_t<DN, DR, 128, GQA>(a, d, stream);
 }
 
 template <int DN>
 void prefill_r(const LatentPrefillArgs& a, const LatentDims& d, hipStream_t stream) {
-    if (d.dr <= 32) prefill_v<DN, 32>(a, d, stream);
-    else prefill_v<DN, 64>(a, d, stream);
+    if (d.dr <= 32) prefill_v<DN, 32, false>(a, d, stream);
+    else prefill_v<DN, 64, false>(a, d, stream);
 }
 
 }  // namespace
@@ -309,6 +334,15 @@ bool launch_latent_prefill(const LatentPrefillArgs& a, const LatentDims& d, hipS
     if (!latent_prefill_supported(d)) return false;
     if (d.dn <= 64) prefill_r<64>(a, d, stream);
     else prefill_r<128>(a, d, stream);
+    return true;
+}
+
+bool gqa_prefill_supported(const LatentDims& d) { return d.dr == 0 && latent_prefill_supported(d); }
+
+bool launch_gqa_prefill(const LatentPrefillArgs& a, const LatentDims& d, hipStream_t stream) {
+    if (!gqa_prefill_supported(d)) return false;
+    if (d.dn <= 64) prefill_v<64, 0, true>(a, d, stream);
+    else prefill_v<128, 0, true>(a, d, stream);
     return true;
 }
 

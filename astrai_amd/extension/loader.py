@@ -96,12 +96,28 @@ def _lightning_attention_module() -> SimpleNamespace:
     return SimpleNamespace(lightning=_mix.lightning, decay_powers=_mix.decay_powers)
 
 
+def _grouped_attention_module() -> SimpleNamespace:
+    return SimpleNamespace(gqa_append=_mix.gqa_append, gqa_prefill=_mix.gqa_prefill, gqa_rows=_mix.gqa_rows)
+
+
+def _gated_recurrence_module() -> SimpleNamespace:
+    return SimpleNamespace(conv=_mix.conv, rglru=_mix.rglru, rglru_step=_mix.rglru_step)
+
+
+def _delta_rule_module() -> SimpleNamespace:
+    return SimpleNamespace(conv=_mix.conv, delta_chunk=_mix.delta_chunk, delta_step=_mix.delta_step)
+
+
 def _residual_rows_module() -> SimpleNamespace:
-    return SimpleNamespace(residual_norm=_mix.residual_norm, embed_norm=_mix.embed_norm, silu_mul=_mix.silu_mul,
-                           gated_rms_norm=_mix.gated_rms_norm)
+    return SimpleNamespace(residual_norm=_mix.residual_norm, embed_norm=_mix.embed_norm, sum_norm=_mix.sum_norm,
+                           act_mul=_mix.act_mul, silu_mul=_mix.silu_mul, gated_rms_norm=_mix.gated_rms_norm,
+                           head_gated_rms_norm=_mix.head_gated_rms_norm)
 
 
 _MIX_FACTORIES = {
+    "delta_rule": _delta_rule_module,
+    "gated_recurrence": _gated_recurrence_module,
+    "grouped_attention": _grouped_attention_module,
     "latent_attention": _latent_attention_module,
     "lightning_attention": _lightning_attention_module,
     "residual_rows": _residual_rows_module,

@@ -3,7 +3,7 @@
 ``StepCache`` is the part every model's cache shares: a capacity, the number of tokens held
 (a host integer that the driver of the steps moves on, since a replayed HIP graph runs no
 Python), and giving it all back. ``MixerCache`` holds whatever the layers of a model with
-different sequence mixers declare: latent rows, recurrent states. ``RequestCaches`` lends
+different sequence mixers declare: rows per position, recurrent states, rings. ``RequestCaches`` lends
 caches to requests and takes them back.
 """
 
@@ -36,11 +36,14 @@ class StepCache:
 
 
 class MixerCache(StepCache):
-    """Per layer, what its mixer carries from token to token:
+    """Per layer, what its mixer carries from token to token. ``slot`` is the layer's number, or (layer, pass)
+    where layers run several times: every pass keeps its own.
 
-      ``latent[i]``  ``[batch, max_len, cols]`` in the model's dtype, one row per position (rows at
-                     or past ``tokens`` are never read, so they need no clearing);
-      ``state[i]``   fp32 ``[batch, ...]``, zero before the first token.
+      ``rows[slot]``   ``[batch, max_len, cols]`` in the model's dtype, one row per position: latents, keys
+                       and values (rows at or past ``tokens`` are never read, so they need no clearing);
+      ``state[slot]``  fp32 ``[batch, ...]``, zero before the first token;
+      ``ring[slot]``   ``[batch, n, cols]`` in the model's dtype, the last inputs of a short convolution, the
+                       one of position p in row p mod n (positions below 0 are not read: no clearing).
 
     ``rotary[key]`` are the rotary tables of the layers' rotations, ``[max_len, pairs, 2]``, one per
     distinct rotation.
@@ -49,15 +52,19 @@ class MixerCache(StepCache):
     def __init__(self, batch: int, max_len: int, device, dtype):
         super().__init__(batch, max_len, device)
         self.dtype = dtype
-        self.latent: Dict[int, Tensor] = {}
-        self.state: Dict[int, Tensor] = {}
+        self.rows: Dict[object, Tensor] = {}
+        self.state: Dict[object, Tensor] = {}
+        self.ring: Dict[object, Tensor] = {}
         self.rotary: Dict[object, Tensor] = {}
 
-    def add_latent(self, layer: int, cols: int) -> None:
-        self.latent[layer] = torch.zeros((self.batch, self.max_len, cols), device=self.device, dtype=self.dtype)
+    def add_rows(self, slot, cols: int) -> None:
+        self.rows[slot] = torch.zeros((self.batch, self.max_len, cols), device=self.device, dtype=self.dtype)
 
-    def add_state(self, layer: int, *shape: int) -> None:
-        self.state[layer] = torch.zeros((self.batch, *shape), device=self.device, dtype=torch.float32)
+    def add_state(self, slot, *shape: int) -> None:
+        self.state[slot] = torch.zeros((self.batch, *shape), device=self.device, dtype=torch.float32)
+
+    def add_ring(self, slot, n: int, cols: int) -> None:
+        self.ring[slot] = torch.zeros((self.batch, n, cols), device=self.device, dtype=self.dtype)
 
     def add_rotary(self, key, build: Callable[..., Tensor]) -> None:
         if key not in self.rotary:

@@ -49,7 +49,7 @@ def load_checkpoint(model_dir: str, device="cuda", dtype: torch.dtype = torch.bf
     arch = architecture_of(config)
     tensors = st.load_file(str(path / _WEIGHTS_FILE))  # safetensors: data only, nothing executed
     with torch.device(device):
-        model = arch.model_class(arch.make_config(config)).to(dtype).eval()
+        model = arch.model_class(arch.configure(config, tensors)).to(dtype).eval()
     return model.load_tensors(tensors)
 
 

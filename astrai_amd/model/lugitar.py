@@ -20,9 +20,8 @@ from torch import Tensor
 
 from astrai_amd.extension import _mix
 from astrai_amd.model.cache import MixerCache
-from astrai_amd.model.decoder import Embedding, Linear
-from astrai_amd.model.mixers import (Fp32Vector, GatedMLP, LatentAttention, LightningAttention, Rotation,
-                                     StepContext, assign_checked)
+from astrai_amd.model.mixers import (Fp32Vector, GatedMLP, LatentAttention, LightningAttention, MixerLM, Rotation,
+                                     assign_checked)
 
 
 @dataclass
@@ -102,81 +101,17 @@ class LugitarLayer(nn.Module):
             self.mlp.load(tensors, prefix + "mlp.")
 
 
-class LugitarLM(nn.Module):
-    """Same calling convention as ``AutoRegressiveLM``: ``model(ids, cache, positions)["logits"]``."""
-
+class LugitarLM(MixerLM):
     def __init__(self, config: LugitarConfig):
-        super().__init__()
-        self.config = config
-        self.embed = Embedding(config.vocab, config.width)
-        self.layers = nn.ModuleList([LugitarLayer(config, i) for i in range(len(config.layers))])
-        self.final_norm = Fp32Vector(config.width)
-        self.head = Linear(config.width, config.vocab)
-        self.apply(lambda m: m.reset_parameters() if hasattr(m, "reset_parameters") else None)
-        self._ready = False
-
-    @property
-    def dtype(self) -> torch.dtype:
-        return self.embed.weight.dtype
-
-    @torch.no_grad()
-    def load_tensors(self, tensors: Dict[str, Tensor]) -> "LugitarLM":
-        """Take every weight from ``tensors`` (stored names); a missing, unknown or misshapen one raises."""
-        left = dict(tensors)
-        cfg = self.config
-        top = assign_checked("model", {"embed": (cfg.vocab, cfg.width), "final.norm": (cfg.width,),
-                                       "head": (cfg.vocab, cfg.width)}, left, "")
-        self.embed.weight.copy_(top["embed"])
-        self.head.weight.copy_(top["head"])
-        self.final_norm.assign(top["final.norm"])
-        for i, layer in enumerate(self.layers):
-            layer.load(left, f"l{i}.")
-        if left:
-            raise ValueError(f"checkpoint does not match the model: unexpected {sorted(left)[:8]}")
-        self._ready = False
-        return self
-
-    def _apply(self, fn, recurse=True):
-        self._ready = False
-        return super()._apply(fn, recurse)
-
-    def finalize(self) -> "LugitarLM":
-        """Derive the weight layouts the kernels read; called by the first forward after loading or
-        moving the model."""
-        for layer in self.layers:
-            layer.mix.finalize()
-        self._ready = True
-        return self
-
-    def new_cache(self, batch: int, max_len: int) -> MixerCache:
-        cache = MixerCache(batch, max_len, self.embed.weight.device, self.dtype)
-        for layer in self.layers:
-            layer.mix.add_to_cache(cache)
-        return cache
+        super().__init__(config, [LugitarLayer(config, i) for i in range(len(config.layers))])
+        self.reset()
 
     @torch.no_grad()
     def forward(self, input_ids: Tensor, kv_cache: Optional[MixerCache] = None, positions: Optional[Tensor] = None,
                 logits_at: Optional[Tensor] = None) -> Dict[str, Tensor]:
-        """``input_ids [batch, seq]``: the tokens after those the cache holds, ``kv_cache.tokens`` of them
-        (``positions``, if given, is those tokens' positions on the device; the caller advances the
-        cache). Without a cache: a sequence of its own. ``logits_at``: indices into the block; only
-        these tokens' logits are formed."""
-        if input_ids.ndim != 2:
-            raise ValueError("input_ids must be [batch, seq_len]")
-        b, s = input_ids.shape
-        if not self._ready:
-            self.finalize()
-        if kv_cache is None:
-            kv_cache = self.new_cache(b, s)
-        if kv_cache.batch != b:
-            raise ValueError(f"{b} sequences with a cache for {kv_cache.batch}")
-        if positions is None:
-            positions = kv_cache.next_positions(s)
-        elif kv_cache.tokens + s > kv_cache.max_len:
-            raise ValueError(f"{s} tokens after {kv_cache.tokens} do not fit a cache of {kv_cache.max_len}")
-        ctx = StepContext(kv_cache, positions, kv_cache.tokens, b, s)
-        cfg, eps, mult = self.config, self.config.eps, self.config.residual_mult
-        n = len(self.layers)
+        """See ``MixerLM.begin``; ``logits_at``: indices into the block; only these tokens' logits are formed."""
+        ctx = self.begin(input_ids, kv_cache, positions)
+        eps, mult = self.config.eps, self.config.residual_mult
         pre = [layer.norm1.weight for layer in self.layers] + [self.final_norm.weight]
         x, h = _mix.embed_norm(self.embed.weight, input_ids.reshape(-1).contiguous(), pre[0], eps)
         for i, layer in enumerate(self.layers):
@@ -186,7 +121,4 @@ class LugitarLM(nn.Module):
             else:
                 h = _mix.residual_norm(y, x, layer.norm1b.weight, layer.norm2.weight, mult, eps)
                 h = _mix.residual_norm(layer.mlp(h), x, layer.norm2b.weight, pre[i + 1], mult, eps)
-        hidden = h.reshape(b, s, cfg.width)
-        if logits_at is not None:
-            hidden = hidden.index_select(1, logits_at)
-        return {"logits": self.head(hidden), "hidden_states": hidden, "residual": x.reshape(b, s, cfg.width)}
+        return self.finish(h, x, ctx, logits_at)

@@ -294,7 +294,7 @@ def test_mix_arguments_are_validated_before_anything_is_launched():
     assert lib.astrai_mix_residual_norm(P, P, P, P, None, P, 4, 8, 1.0, 1e-6, 0, None) == 1 and "null" in err()
     assert lib.astrai_mix_residual_norm(P, P, P, 8, P, P, 4, 8, 1.0, 1e-6, 0, None) == 1 and "aligned" in err()
     assert lib.astrai_mix_residual_norm(P, P, P, P, P, P, 4, 8, 1.0, 1e-6, 7, None) == 1 and "dtype" in err()
-    assert lib.astrai_mix_silu_mul(P, P, 4, 12, 0, None) == 1
+    assert lib.astrai_mix_act_mul(P, P, 4, 12, 0, 0, None) == 1
     assert lib.astrai_mix_gated_rms_norm(P, P, 8, P, P, 4, 16, 16, 1e-6, 0, None) == 1
     tail = (1, 8, 64, 3, 32, 32, 64, 56, 1e-6, 0, None)   # batch, seq, max_len, heads, dn, dr, rp, kv_rank
     assert lib.astrai_mix_latent_append(P, 200, 192, P, 64, 4, P, P, P, None, None, *tail) == 1 and "row stride" in err()
