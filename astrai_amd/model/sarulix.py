@@ -23,7 +23,7 @@ from torch import Tensor
 from astrai_amd.extension import _mix
 from astrai_amd.model.cache import MixerCache
 from astrai_amd.model.mixers import (ChannelDelta, Fp32Vector, GatedMLP, GatedRecurrence, GroupedAttention, MixerLM,
-                                     PackedLinear, Rotation, Rows, assign_checked, linear_f32)
+                                     PackedLinear, Rotation, Rows, assign_checked, columns_of, linear_f32)
 
 NO_LOOP = (0, 0, 0)
 
@@ -140,8 +140,7 @@ class SarulixLM(MixerLM):
         # W_in: W_a (on x), then W_b (on x0)
         self.loop_in = self.loop_step = None
         if config.loop != NO_LOOP:
-            whole = Rows("x", 1, ((w, w),))
-            self.loop_in = PackedLinear(whole, [Rows("a", 1, ((w, w),)), Rows("b", 1, ((w, w),))])
+            self.loop_in = PackedLinear(Rows("x", 1, ((w, w),)), [columns_of("a", w), columns_of("b", w)])
             self.loop_step = nn.ModuleList([Fp32Vector(w) for _ in range(config.loop[2])])
         self.reset()
 
@@ -176,17 +175,17 @@ class SarulixLM(MixerLM):
                              mult=cfg.embedding_scale)
         u = None
         if self.loop_in is not None:
-            w_a, w_b = self.loop_in.weight[:w], self.loop_in.weight[w:]
+            b = self.loop_in.offset["b"]
             if not order[0][2]:
-                u = linear_f32(x.to(dtype), w_b)
+                u = linear_f32(x.to(dtype), self.loop_in.weight[b:])[:, :w]
         for k, (i, ctx.run, begins) in enumerate(order):
             layer = self.layers[i]
             if begins:
                 if u is None:
                     both = linear_f32(h, self.loop_in.weight)
-                    y, u = both[:, :w], both[:, w:]
+                    y, u = both[:, :w], both[:, b:b + w]
                 else:
-                    y = linear_f32(h, w_a)
+                    y = linear_f32(h, self.loop_in.weight[:b])[:, :w]
                 _, h = _mix.sum_norm(y, layer.norm1.weight, dtype, eps, u=u, vec=self.loop_step[ctx.run].weight, out=x)
             y = layer.mix(h, ctx)
             if layer.mlp is not None:

@@ -339,14 +339,119 @@ def _lugitar_kernels(dev, width, heads, ff, batch, seq, window=1024):
     return res
 
 
-def _bench_lugitar(dev):
-    """Lugitar models (random weights, bf16) beside the dense GQA decoder of equal width, depth and feed-forward,
-    in its own bf16 form and in its fused int8 form: prompt and decode throughput, then the kernels."""
+def _sarulix_config(width, heads, ff, layers, vocab=32000):
+    """A Sarulix model with layers of a real model's sizes: groups of four layers (gated recurrence, delta rule,
+    gated recurrence, attention with four query heads per key/value head), heads of 128, blocks of 256 channels; the
+    middle third runs twice, ``layers`` layer runs in all."""
+    distinct = layers * 3 // 4
+    start = (distinct - layers // 4) // 2
+    out = []
+    for i in range(distinct):
+        kind = ("rglru", "channel_delta", "rglru", "attention")[i % 4]
+        mixer = {"rglru": {"width": width, "blocks": width // 256, "conv": 4},
+                 "channel_delta": {"heads": heads, "kv_heads": heads, "dim": 128, "vdim": 128, "conv": 4},
+                 "attention": {"heads": heads, "kv_heads": heads // 4, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                               "softcap": 50.0, "rot": {"dims": 64, "base": 10000.0}}}[kind]
+        out.append({"type": kind, "mixer": mixer, "mlp": {"kind": "dense", "ff": ff}})
+    return {"architecture": "Sarulix", "vocab": vocab, "width": width, "layers": out, "norm": {"eps": 1e-6},
+            "embedding": {"scale": 1.0}, "logit_scale": 1.0,
+            "loop": {"start": start, "stop": start + layers // 4, "times": 2}}
+
+
+def _sarulix_kernels(dev, width, heads, ff, batch, seq, ctx=1024):
+    """Every kernel of a Sarulix layer beside the like kernel of the dense decoder or of Lugitar at equal size; as
+    ``_lugitar_kernels``."""
+    import torch
+
+    from astrai_amd.extension import _cabi, _mix
+
+    bf, f32 = torch.bfloat16, torch.float32
+    n, hkv, d = batch * seq, heads // 4, 128
+    hd, w, bp, taps = heads * d, width, 256, 4
+    blocks, most = width // 256, max(ctx, seq)
+    res = {}
+
+    def r(*size, dtype=bf, scale=1.0):
+        return (torch.randn(*size, device=dev) * scale).to(dtype)
+
+    def entry(name, fn, nbytes, flops=0.0, launches=20):
+        us = _graph_us(lambda i: fn(), launches)
+        roof = max(nbytes / (PEAK_HBM_GBS * 1e9), flops / (PEAK_BF16_TFLOPS * 1e12)) * 1e6
+        res[name] = {"us": round(us, 2), "roofline": round(roof / us, 3)}
+
+    causal = seq * (seq + 1) / 2
+    pos, last = torch.arange(seq, device=dev), torch.tensor([ctx - 1], device=dev)
+    # --- attention
+    s = _mix.GqaShape(heads, hkv, d, d, d, d ** -0.5, 50.0, True)
+    q, kc, vc = r(batch, heads, seq, d), r(batch, hkv, most, d), r(batch, hkv, most, d)
+    entry("dense attn_prefill", lambda: _cabi.attn_prefill(q, kc, vc, pos),
+          (2 * n * hd + 2 * n * hkv * d) * 2, 4 * d * heads * batch * causal)
+    cols = 2 * hd + 2 * hkv * d
+    proj, cache = r(n, cols), r(batch, most, s.cache_cols)
+    entry("gqa_prefill", lambda: _mix.gqa_prefill(proj, s, cols - hd, cache, 0),
+          (3 * n * hd + 2 * n * hkv * d) * 2, 4 * d * heads * batch * causal)
+    q1, kc1, vc1, p1 = r(batch, heads, 1, d), r(batch, hkv, ctx, d), r(batch, hkv, ctx, d), r(batch, cols)
+    entry("dense attn_decode", lambda: _cabi.attn_decode(q1, kc1, vc1, last), 2 * batch * hkv * ctx * d * 2)
+    entry("gqa_rows", lambda: _mix.gqa_rows(p1, s, cols - hd, cache, last, True), 2 * batch * hkv * ctx * d * 2)
+    # --- recurrences, prompt: chunked lightning as the like kernel
+    lproj, lstate = r(n, 4 * hd), torch.zeros(batch, heads, d, d, device=dev)
+    dec = _mix.decay_powers([0.5 + 0.49 * h / heads for h in range(heads)]).to(dev)
+    entry("lightning chunk", lambda: _mix.lightning(lproj, 0, hd, 2 * hd, dec, lstate, False),
+          4 * n * hd * 2 + 2 * lstate.numel() * 4, n * heads * 2 * (32 * d + 32 * d + 2 * d * d))
+    entry("lightning step", lambda: _mix.lightning(lproj[:batch], 0, hd, 2 * hd, dec, lstate, True), 2 * lstate.numel() * 4)
+    yx, u = r(n, 2 * w), r(n, w)
+    wr, wi = r(blocks, bp, bp, scale=bp ** -0.5), r(blocks, bp, bp, scale=bp ** -0.5)
+    zero, coef = torch.zeros(w, device=dev), torch.full((w,), -1.0, device=dev)
+    state, cw = torch.zeros(batch, w, device=dev), r(taps, w, dtype=f32)
+    ring = torch.zeros(batch, _mix.ring_rows(taps), w, device=dev, dtype=bf)
+    gates = (wr, wi, zero, zero, coef, state)
+    entry("rglru chunk", lambda: _mix.rglru(u, yx, 0, *gates, matrix=True), 3 * n * w * 2, 4 * n * w * bp)
+    entry("rglru step", lambda: _mix.rglru_step(yx[:batch], 0, w, cw, zero, ring, last, *gates),
+          batch * w * (3 * 2 + taps * 2 + 8) + 2 * wr.numel() * 2)
+    ds = _mix.DeltaShape(heads, heads, d, d, d, d ** -0.5)
+    dcols = 3 * hd + heads
+    dproj, qkv, z = r(n, dcols), r(n, 3 * hd), r(n, hd, dtype=f32)
+    dtb, one, gate, nw = torch.full((hd,), -4.0, device=dev), torch.ones(heads, device=dev), r(n, hd), torch.ones(d, device=dev)
+    dcw = r(taps, 3 * hd, dtype=f32, scale=0.5)
+    dring = torch.zeros(batch, _mix.ring_rows(taps), 3 * hd, device=dev, dtype=bf)
+    entry("delta chunk", lambda: _mix.delta_chunk(qkv, dproj, ds, 3 * hd, z, dtb, one, lstate),
+          n * hd * (3 * 2 + 4 + 2) + 2 * lstate.numel() * 4, n * heads * 2 * (3 * d * d + 32 * d))
+    entry("delta step", lambda: _mix.delta_step(dproj[:batch], ds, 3 * hd, z[:batch], dtb, one, gate[:batch], nw, lstate, 1e-6,
+                                                x_off=0, conv_w=dcw, ring=dring, positions=last),
+          2 * lstate.numel() * 4 + batch * hd * (3 * 2 * (1 + taps) + 4 + 2 + 2))
+    # --- row operations, prompt and decode
+    for tag, rows in (("prefill", n), ("decode", batch)):
+        y, xf, w32 = r(rows, width), r(rows, width, dtype=f32), torch.ones(width, device=dev)
+        entry(f"residual_norm {tag}", lambda: _mix.residual_norm(y, xf, w32, w32, 0.5, 1e-6), rows * width * (2 + 4 + 4 + 2))
+        entry(f"sum_norm {tag}", lambda: _mix.sum_norm(y, w32, bf, 1e-6, x=xf, out=xf), rows * width * (2 + 4 + 4 + 2))
+        gu = r(rows, 2 * ff)
+        entry(f"silu_mul {tag}", lambda: _mix.silu_mul(gu), rows * ff * 6)
+        entry(f"act_mul gelu {tag}", lambda: _mix.act_mul(gu, "gelu_tanh"), rows * ff * 6)
+        o, wv = r(rows, hd), torch.ones(hd, device=dev)
+        entry(f"gated_rms_norm {tag}", lambda: _mix.gated_rms_norm(o, lproj[:rows], 3 * hd, wv, hd, 1e-6), rows * hd * 6)
+        if tag == "prefill":
+            entry("head_gated_rms_norm", lambda: _mix.head_gated_rms_norm(o, gate, nw, d, 1e-6), rows * hd * 6)
+            entry("conv of one tensor", lambda: _mix.conv(yx, w, cw, zero, ring, pos, False), rows * w * 4)
+            entry("conv + silu of q, k, v", lambda: _mix.conv(dproj, 0, dcw, None, dring, pos, True), rows * hd * 12)
+        s1 = rows // batch
+        kv, fr = r(batch, s1, (heads + 2 * hkv) * d), r(s1, d // 2, 2, dtype=f32)
+        ps = torch.arange(s1, device=dev)
+        entry(f"dense rope_cache_write {tag}", lambda: _cabi.rope_cache_write(kv, fr, ps, kc, vc, heads, hkv, d),
+              2 * kv.numel() * 2)
+        rot, dn = r(most, 32, 2, dtype=f32), torch.ones(d, device=dev)
+        pj = proj[:rows]
+        entry(f"gqa_append {tag}", lambda: _mix.gqa_append(pj, s, hd, hd + hkv * d, rot, ps, dn, dn, cache, 1e-6),
+              2 * kv.numel() * 2)
+    return res
+
+
+def _bench_designs(dev, designs, cases, kernel_cases, kernels):
+    """Models of several designs at equal width, depth and feed-forward (random weights): prompt and decode throughput,
+    then the kernels. ``designs``: tag -> (builds the model of a case, context it runs under)."""
     import torch
 
     from astrai_amd.extension import w8a8
-    from astrai_amd.model import (AutoRegressiveLM, AutoRegressiveLMConfig, LugitarConfig, LugitarLM,
-                                  fuse_int8_weights, greedy_generate)
+    from astrai_amd.model import greedy_generate
 
     def timed(fn, reps=3):
         for _ in range(2):
@@ -361,15 +466,15 @@ def _bench_lugitar(dev):
         return sorted(ts)[len(ts) // 2]
 
     out = {"models": [], "kernels": []}
-    cases = [(2048, 16, 5632, 24, 32, 512, 64), (2048, 16, 5632, 24, 1, 4096, 64), (4096, 32, 8192, 8, 8, 2048, 64)]
     for width, heads, ff, layers, batch, prompt, steps in cases:
         row = {"width": width, "layers": layers, "ff": ff, "heads": heads, "batch": batch, "prompt": prompt}
         ids = torch.randint(0, 32000, (batch, prompt), generator=torch.Generator().manual_seed(4)).to(dev)
-
-        def legs(tag, model):
-            with torch.no_grad():
-                last = torch.tensor([prompt - 1], device=dev)
-
+        last = torch.tensor([prompt - 1], device=dev)
+        for tag, (build, context) in designs.items():
+            torch.manual_seed(5)
+            with torch.device(dev):
+                model = build(width, heads, ff, layers, prompt + 2 * steps)
+            with torch.no_grad(), context():
                 def prefill():
                     return model(ids, model.new_cache(batch, prompt + steps), logits_at=last)["logits"]
 
@@ -383,33 +488,71 @@ def _bench_lugitar(dev):
                 row[tag] = {"prefill_ms": round(t_pre * 1e3, 2), "prefill_tokens_per_s": round(batch * prompt / t_pre),
                             "decode_ms_per_step": round(step * 1e3, 3),
                             "decode_tokens_per_s": round(batch / step), "generate_1_ms": round(t_gen0 * 1e3, 2)}
-
-        torch.manual_seed(5)
-        with torch.device(dev):
-            model = LugitarLM(LugitarConfig.from_dict(_lugitar_config(width, heads, ff, layers))).to(torch.bfloat16).eval()
-        legs("lugitar_bf16", model)
-        del model
-        cfg = AutoRegressiveLMConfig(hidden_size=width, num_hidden_layers=layers, num_attention_heads=heads,
-                                     num_key_value_heads=heads // 4, intermediate_size=ff,
-                                     max_position_embeddings=prompt + 2 * steps)
-        with torch.device(dev):
-            model = AutoRegressiveLM(cfg).to(torch.bfloat16).eval()
-        legs("dense_bf16", model)
-        w8a8.int8_state().reset()
-        fuse_int8_weights(model)
-        with w8a8.int8_autocast(True):
-            legs("dense_fused_int8", model)
-        w8a8.int8_state().reset()
-        del model
-        torch.cuda.empty_cache()
+            del model
+            w8a8.int8_state().reset()
+            torch.cuda.empty_cache()
         out["models"].append(row)
         print(json.dumps(row), file=sys.stderr, flush=True)
-    for width, heads, ff, batch, seq in ((2048, 16, 5632, 32, 512), (4096, 32, 8192, 4, 4096)):
+    for width, heads, ff, batch, seq in kernel_cases:
         k = {"width": width, "heads": heads, "ff": ff, "batch": batch, "seq": seq,
-             "kernels": _lugitar_kernels(dev, width, heads, ff, batch, seq)}
+             "kernels": kernels(dev, width, heads, ff, batch, seq)}
         out["kernels"].append(k)
         print(json.dumps(k), file=sys.stderr, flush=True)
     return out
+
+
+MODEL_CASES = [(2048, 16, 5632, 24, 32, 512, 64), (2048, 16, 5632, 24, 1, 4096, 64), (4096, 32, 8192, 8, 8, 2048, 64)]
+KERNEL_CASES = [(2048, 16, 5632, 32, 512), (4096, 32, 8192, 4, 4096)]
+
+
+def _dense_model(width, heads, ff, layers, positions):
+    import torch
+
+    from astrai_amd.model import AutoRegressiveLM, AutoRegressiveLMConfig
+    cfg = AutoRegressiveLMConfig(hidden_size=width, num_hidden_layers=layers, num_attention_heads=heads,
+                                 num_key_value_heads=heads // 4, intermediate_size=ff,
+                                 max_position_embeddings=positions)
+    return AutoRegressiveLM(cfg).to(torch.bfloat16).eval()
+
+
+def _lugitar_model(width, heads, ff, layers, positions):
+    import torch
+
+    from astrai_amd.model import LugitarConfig, LugitarLM
+    return LugitarLM(LugitarConfig.from_dict(_lugitar_config(width, heads, ff, layers))).to(torch.bfloat16).eval()
+
+
+def _sarulix_model(width, heads, ff, layers, positions):
+    import torch
+
+    from astrai_amd.model import SarulixConfig, SarulixLM
+    return SarulixLM(SarulixConfig.from_dict(_sarulix_config(width, heads, ff, layers))).to(torch.bfloat16).eval()
+
+
+def _bench_lugitar(dev):
+    """Lugitar models (bf16) beside the dense GQA decoder in its own bf16 form and in its fused int8 form."""
+    from contextlib import nullcontext
+
+    from astrai_amd.extension import w8a8
+    from astrai_amd.model import fuse_int8_weights
+
+    def fused(*case):
+        model = _dense_model(*case)
+        fuse_int8_weights(model)
+        return model
+
+    designs = {"lugitar_bf16": (_lugitar_model, nullcontext), "dense_bf16": (_dense_model, nullcontext),
+               "dense_fused_int8": (fused, lambda: w8a8.int8_autocast(True))}
+    return _bench_designs(dev, designs, MODEL_CASES, KERNEL_CASES, _lugitar_kernels)
+
+
+def _bench_sarulix(dev):
+    """Sarulix models (bf16) beside Lugitar and the dense GQA decoder in bf16."""
+    from contextlib import nullcontext
+
+    designs = {"sarulix_bf16": (_sarulix_model, nullcontext), "lugitar_bf16": (_lugitar_model, nullcontext),
+               "dense_bf16": (_dense_model, nullcontext)}
+    return _bench_designs(dev, designs, MODEL_CASES, KERNEL_CASES, _sarulix_kernels)
 
 
 def _cpu_decoder_baseline(layers=1, prefill_batch=8, decode_steps=8):
@@ -569,6 +712,11 @@ def main():
     ap.add_argument("--lugitar-trace", action="store_true",
                     help="tracing mode: an 8-layer Lugitar model, one 32 x 512-token prompt + 7 eager decode steps, "
                          "nothing else")
+    ap.add_argument("--sarulix", action="store_true",
+                    help="Sarulix models beside Lugitar and the dense decoder of equal size, and every kernel beside "
+                         "its like; prints one JSON line of its own")
+    ap.add_argument("--sarulix-trace", action="store_true",
+                    help="tracing mode: --lugitar-trace for a Sarulix model of 8 layer runs")
     ap.add_argument("--pmc", action="store_true",
                     help="counter-collection mode: a few launches of the headline kernel and of a "
                          "plain 256 MiB device copy (the calibration kernel), nothing else")
@@ -578,7 +726,7 @@ def main():
                  "(no multi-GPU leg exists: the path shards by output columns or by K, one collective at most)")
 
     tracing = bool(args.decoder_trace or args.trace_kernels or args.trace_gemms or args.pmc or args.lugitar
-                   or args.lugitar_trace)
+                   or args.lugitar_trace or args.sarulix or args.sarulix_trace)
     ceilings = {} if tracing else _measured_ceilings()
 
     import torch
@@ -601,16 +749,20 @@ def main():
     if args.lugitar:
         print(json.dumps({"lugitar": _bench_lugitar(dev)}))
         return
-    if args.lugitar_trace:
-        from astrai_amd.model import LugitarConfig, LugitarLM, greedy_generate
+    if args.sarulix:
+        print(json.dumps({"sarulix": _bench_sarulix(dev)}))
+        return
+    if args.lugitar_trace or args.sarulix_trace:
+        from astrai_amd.model import greedy_generate
 
+        name, build = ("lugitar", _lugitar_model) if args.lugitar_trace else ("sarulix", _sarulix_model)
         torch.manual_seed(5)
         with torch.device(dev):
-            model = LugitarLM(LugitarConfig.from_dict(_lugitar_config(2048, 16, 5632, 8))).to(torch.bfloat16).eval()
+            model = build(2048, 16, 5632, 8, 520)
         ids = torch.randint(0, 32000, (32, 512), generator=torch.Generator().manual_seed(4)).to(dev)
         greedy_generate(model, ids, 8)
         torch.cuda.synchronize()
-        print(json.dumps({"lugitar_trace": "8 layers", "prompt_tokens": 32 * 512, "decode_steps": 7}))
+        print(json.dumps({f"{name}_trace": "8 layers", "prompt_tokens": 32 * 512, "decode_steps": 7}))
         return
 
     if args.decoder_trace:
