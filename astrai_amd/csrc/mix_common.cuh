@@ -81,18 +81,6 @@ __device__ __forceinline__ float gelu_as(float z) {
     return z * (sizeof(T) == 2 ? sigmoid_fast(y2) : sigmoid(y2));
 }
 
-// 1 - e^x for x <= 0 given ex = e^x: a Taylor polynomial where the difference would cancel
-__device__ __forceinline__ float one_minus_exp(float x, float ex) {
-    float p = 1.0f + x * (1.0f / 8.0f);
-    p = 1.0f + x * (1.0f / 7.0f) * p;
-    p = 1.0f + x * (1.0f / 6.0f) * p;
-    p = 1.0f + x * (1.0f / 5.0f) * p;
-    p = 1.0f + x * (1.0f / 4.0f) * p;
-    p = 1.0f + x * (1.0f / 3.0f) * p;
-    p = 1.0f + x * (1.0f / 2.0f) * p;
-    return x > -0.35f ? -x * p : 1.0f - ex;
-}
-
 // log(1 + e^z): max(z, 0) + log(1 + e), e = e^-|z| in (0, 1]; a Taylor polynomial for small e, where 1 + e
 // would drop its digits
 __device__ __forceinline__ float softplus_fast(float z) {

@@ -11,7 +11,7 @@
 //          (the "image"). L cannot be split into a factor of t and one of j against the chunk's start (the
 //          second would overflow under strong decays), so pairs are grouped by the highest bit in which t
 //          and j differ: with m the middle of their common block of 2, 4, 8 or 16 tokens, L_tj is
-//          (decays m .. t)(decays j + 1 .. m - 1), both <= 1. One wave per such level, one MFMA product each.
+//          (decays m .. t)(decays j + 1 .. m - 1), both <= 1. One wave per such level and product.
 //   walk   chunk after chunk per head; a wave owns 16 or 32 value columns and all key channels, S in fp32
 //          accumulators. With value columns as MFMA columns throughout, every accumulator (S, V - Y, U) is
 //          the next product's operand already; images stream into LDS by direct loads, one chunk ahead.
@@ -20,6 +20,8 @@
 //
 // Step kernel (decoding, and everything in float): token by token, the state in registers, one workgroup per
 // head; norm and output gate in its epilogue. For a few tokens it also convolves its inputs.
+#include <type_traits>
+
 #include "mix_conv.cuh"
 #include "mix_launchers.h"
 
@@ -204,21 +206,20 @@ __device__ __forceinline__ u32x4 split4(f32x4 v) {   // four high terms, four lo
     return u32x4{h0, h1, l0, l1};
 }
 
-__device__ __forceinline__ void put_split(uint8_t* hi, uint8_t* lo, int off, float v) {
-    uint32_t h, l;
-    split2(v, 0.0f, h, l);
-    *reinterpret_cast<uint16_t*>(hi + off) = (uint16_t)h;
-    *reinterpret_cast<uint16_t*>(lo + off) = (uint16_t)l;
-}
+constexpr int kPrepThreads = 512;
 
+// Thread roles: a pair of channels, keys or queries, eight of the 16 tokens, one of two levels at a time. A level's
+// matrices hold the factors of keys for all tokens and of queries for the upper ones; the levels are done in two rounds
+// of two, so that four workgroups fit a CU.
 template <int DP>
-__global__ __launch_bounds__(256) void delta_prep_kernel(DeltaArgs a, int chunks) {
+__global__ __launch_bounds__(kPrepThreads, DP <= 128 ? 8 : 2) void delta_prep_kernel(DeltaArgs a, int chunks) {
     constexpr int NS = DP / 32, kRow = DP * 2 + 16, kMat = kC * kRow;   // bytes
-    constexpr int kPer = (DP + 127) / 128;        // channels per thread
+    constexpr int kPairs = DP / 2, kPer = (kPairs + 63) / 64;           // channel pairs, of a thread
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
-    uint8_t* const mats = lds;                    // [4 levels][k hi, k lo, q hi, q lo][kC][kRow]
-    float* const lg = reinterpret_cast<float*>(lds + 16 * kMat);   // [kC][DP] decays
-    float* const inv = lg + kC * DP;              // [2][kC]: factor of q, of k
+    constexpr int kHalfMat = kMat / 2, kLevel = 2 * kMat + 2 * kHalfMat;
+    uint8_t* const mats = lds;                    // [2 levels][k hi, k lo: kC rows; q hi, q lo: kC / 2 rows][kRow]
+    float* const lg = reinterpret_cast<float*>(lds + 2 * kLevel);   // [kC][DP] decays
+    float* const inv = lg + kC * DP;              // [2][kC]: factor of k, of q
     float* const diag = inv + 2 * kC;             // [kC]
     float* const beta = diag + kC;                // [kC]
     float* const ms = beta + kC;                  // [kC][20]
@@ -232,8 +233,8 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(DeltaArgs a, int chunks
     const uint16_t* k = q + a.kv_heads * a.dp;
     uint8_t* image = static_cast<uint8_t*>(a.image) + (((int64_t)b * a.heads + h) * chunks + chunk) * (Image<DP>::kDma * 1024);
 
-    // norms: 16 lanes per token, which also give q . k of the same token
-    {
+    // the first half: norms, 16 lanes per token, which also give q . k of the same token
+    if (wave < 4) {
         const int t = tid >> 4, l = tid & 15;
         float sq = 0.0f, sk = 0.0f, qk = 0.0f;
         if (t < n)
@@ -256,135 +257,191 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(DeltaArgs a, int chunks
         }
         if (l == 0) {
             const float fq = a.q_scale / sqrtf(sq + kUnitEps), fk = 1.0f / sqrtf(sk + kUnitEps);
-            inv[t] = fq;
-            inv[kC + t] = fk;
+            inv[t] = fk;
+            inv[kC + t] = fq;
             diag[t] = qk * fq * fk;
             beta[t] = t < n ? sigmoid(Elem<uint16_t>::get(static_cast<const uint16_t*>(a.proj) + (row0 + t) * a.ld + a.b_off + h))
                             : 0.0f;
         }
     }
-    // decays: each half of the workgroup eight tokens
+    // decays, four channels at a time
     {
-        const float decay = a.decay[h];
-        const int half = tid >> 7;
-        for (int d = tid & 127; d < DP; d += 128) {
-            const float bias = d < a.dp ? a.dt_bias[h * a.dp + d] : 0.0f;
+        const float decay = -kLog2e * a.decay[h];
+        const float* z = a.z + row0 * a.heads * a.dp + h * a.dp;
+        for (int i = tid; i < kC * (DP / 4); i += kPrepThreads) {
+            const int t = i / (DP / 4), d = i % (DP / 4) * 4;
+            f32x4 x = {1, 1, 1, 1};
+            if (t < n && d < a.dp) {
+                const f32x4 zz = *reinterpret_cast<const f32x4*>(z + (int64_t)t * a.heads * a.dp + d);
+                const f32x4 bias = *reinterpret_cast<const f32x4*>(a.dt_bias + h * a.dp + d);
 #pragma unroll
-            for (int i = 0; i < 8; ++i) {
-                const int t = half * 8 + i;
-                float x = 1.0f;
-                if (t < n && d < a.dp)
-                    x = __builtin_amdgcn_exp2f(-kLog2e * decay * softplus_fast(a.z[(row0 + t) * a.heads * a.dp + h * a.dp + d] + bias));
-                lg[t * DP + d] = x;
+                for (int e = 0; e < 4; ++e) x[e] = __builtin_amdgcn_exp2f(decay * softplus_fast(zz[e] + bias[e]));
             }
+            *reinterpret_cast<f32x4*>(lg + t * DP + d) = x;
+        }
+    }
+    const bool is_q = wave >= 4;
+    const int half = wave & 1, sel = (wave >> 1) & 1, r0 = half * 8;   // tokens r0 .. r0 + 7
+    f32x2 x[kPer][8];    // this pair's unit vectors
+    const uint16_t* src = is_q ? q : k;
+#pragma unroll
+    for (int p = 0; p < kPer; ++p) {
+        const int d = (lane + p * 64) * 2;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+            const int t = r0 + i;
+            const uint32_t raw = (t < n && d < a.dp) ? *reinterpret_cast<const uint32_t*>(src + (int64_t)t * a.ldq + d) : 0;
+            x[p][i] = f32x2{__uint_as_float(raw << 16), __uint_as_float(raw & 0xffff0000u)};
         }
     }
     __syncthreads();
-    // operands: half 0 the keys, half 1 the queries, a channel per thread
-    {
-        const bool is_q = tid >= 128;
-        const uint16_t* src = is_q ? q : k;
-        const float* f = inv + (is_q ? 0 : kC);
+    auto scale = [](f32x2 u, f32x2 v) { return f32x2{u[0] * v[0], u[1] * v[1]}; };
+    // both terms of a pair, the low ones `dist` bytes further
+    auto put = [&](uint8_t* hi, int dist, int off, f32x2 v) {
+        uint32_t h2, l2;
+        split2(v[0], v[1], h2, l2);
+        *reinterpret_cast<uint32_t*>(hi + off) = h2;
+        *reinterpret_cast<uint32_t*>(hi + dist + off) = l2;
+    };
+#pragma unroll
+    for (int p = 0; p < kPer; ++p)
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+            const float f = inv[(is_q ? kC : 0) + r0 + i];
+            x[p][i] = scale(x[p][i], f32x2{f, f});
+        }
+#pragma unroll
+    for (int round = 0; round < 2; ++round) {
+        if (round) __syncthreads();   // the first round's matrices are no longer read
+        uint8_t* const lv = mats + sel * kLevel;
 #pragma unroll
         for (int p = 0; p < kPer; ++p) {
-            const int d = (tid & 127) + p * 128;
-            if (d < DP) {
-                float x[kC], dec[kC];
+            const int d = (lane + p * 64) * 2;
+            if (d >= DP) continue;
+            f32x2 dec[8];
 #pragma unroll
-                for (int t = 0; t < kC; ++t) {
-                    x[t] = (t < n && d < a.dp) ? Elem<uint16_t>::get(src + (int64_t)t * a.ldq + d) * f[t] : 0.0f;
-                    dec[t] = lg[t * DP + d];
+            for (int i = 0; i < 8; ++i) dec[i] = *reinterpret_cast<const f32x2*>(lg + (r0 + i) * DP + d);
+            // Tokens M .. M + HB - 1 of this half as a block's upper ones: they take the decays M .. t. Their rank
+            // among the level's upper tokens is the row of a query.
+            auto upper = [&](auto hb, auto m) {
+                f32x2 w = {1.0f, 1.0f};
+#pragma unroll
+                for (int i = m; i < m + hb; ++i) {
+                    w = scale(w, dec[i]);
+                    const f32x2 v = scale(x[p][i], w);
+                    const int t = r0 + i, rank = (t / (2 * hb)) * hb + t % hb;
+                    if (is_q) put(lv + 2 * kMat, kHalfMat, rank * kRow + d * 2, v);
+                    else put(lv, kMat, t * kRow + d * 2, v);
                 }
-                // levels: blocks of 2 hb tokens, middle m; upper tokens take decays m .. t, lower ones j + 1 .. m - 1
+            };
+            // the HB tokens before the middle M as its lower ones (keys): decays j + 1 .. M - 1
+            auto lower = [&](auto hb, auto m) {
+                if (is_q) return;
+                f32x2 w = {1.0f, 1.0f};
 #pragma unroll
-                for (int lv = 0; lv < 4; ++lv) {
-                    constexpr int kHalf[4] = {8, 4, 2, 1};
-                    const int hb = kHalf[lv];
-                    uint8_t* hi = mats + (lv * 4 + (is_q ? 2 : 0)) * kMat;
-                    uint8_t* lo = hi + kMat;
-#pragma unroll
-                    for (int m = hb; m < kC; m += 2 * hb) {
-                        float w = 1.0f;
-#pragma unroll
-                        for (int t = m; t < m + hb; ++t) {
-                            w *= dec[t];
-                            put_split(hi, lo, t * kRow + d * 2, x[t] * w);
-                        }
-                        if (!is_q) {
-                            w = 1.0f;
-#pragma unroll
-                            for (int j = m - 1; j >= m - hb; --j) {
-                                put_split(hi, lo, j * kRow + d * 2, x[j] * w);
-                                w *= dec[j];
-                            }
-                        }
-                    }
+                for (int i = m - 1; i >= m - hb; --i) {
+                    put(lv, kMat, (r0 + i) * kRow + d * 2, scale(x[p][i], w));
+                    w = scale(w, dec[i]);
                 }
-                // G K, G Q: into the image, channels in the order of the accumulators' rows
-                {
-                    const int s = d >> 5, r = d & 31, pos = ((r & 15) >> 2) * 8 + (r >> 4) * 4 + (r & 3);   // 8 gg + j
-                    uint8_t* hi = image + ((is_q ? 2 * NS : 0) + s) * 1024 + (pos >> 3) * 256 + (pos & 7) * 2;
-                    uint8_t* lo = hi + NS * 1024;
-                    float w = 1.0f;
-#pragma unroll
-                    for (int t = 0; t < kC; ++t) {
-                        w *= dec[t];
-                        put_split(hi, lo, t * 16, x[t] * w);
-                    }
-                    if (!is_q) reinterpret_cast<float*>(image + Image<DP>::kFrags * 1024)[d] = w;
+            };
+            using std::integral_constant;
+            auto block = [&](auto hb, auto m) {
+                lower(hb, m);
+                upper(hb, m);
+            };
+            if (round == 0) {
+                if (sel == 0) {
+                    if (half) upper(integral_constant<int, 8>{}, integral_constant<int, 0>{});
+                    else lower(integral_constant<int, 8>{}, integral_constant<int, 8>{});
+                } else {
+                    block(integral_constant<int, 4>{}, integral_constant<int, 4>{});
                 }
-                if (!is_q) {
-                    float w = 1.0f;
+            } else if (sel == 0) {
+                block(integral_constant<int, 2>{}, integral_constant<int, 2>{});
+                block(integral_constant<int, 2>{}, integral_constant<int, 6>{});
+            } else {
+                block(integral_constant<int, 1>{}, integral_constant<int, 1>{});
+                block(integral_constant<int, 1>{}, integral_constant<int, 3>{});
+                block(integral_constant<int, 1>{}, integral_constant<int, 5>{});
+                block(integral_constant<int, 1>{}, integral_constant<int, 7>{});
+            }
+            // the last key parts: L_15 K straight into the image
+            if (round == sel && !is_q && sel == 1) {
+                f32x2 w = {1.0f, 1.0f};
+                if (!half) {
 #pragma unroll
-                    for (int j = kC - 1; j >= 0; --j) {
-                        x[j] *= w;
-                        w *= dec[j];
-                    }
-                    uint8_t* dst = image + (4 * NS + (d >> 4)) * 1024 + (d & 15) * 16;
-#pragma unroll
-                    for (int gg = 0; gg < 4; ++gg)
-                        *reinterpret_cast<u32x4*>(dst + gg * 256) = split4(f32x4{x[4 * gg], x[4 * gg + 1], x[4 * gg + 2], x[4 * gg + 3]});
+                    for (int t = kC - 1; t >= 8; --t) w = scale(w, *reinterpret_cast<const f32x2*>(lg + t * DP + d));
                 }
+                f32x2 v[8];
+#pragma unroll
+                for (int i = 7; i >= 0; --i) {
+                    v[i] = scale(x[p][i], w);
+                    w = scale(w, dec[i]);
+                }
+                uint8_t* dst = image + (4 * NS + (d >> 4)) * 1024 + (d & 15) * 16 + half * 512;
+#pragma unroll
+                for (int gg = 0; gg < 2; ++gg)
+#pragma unroll
+                    for (int e = 0; e < 2; ++e)
+                        *reinterpret_cast<u32x4*>(dst + gg * 256 + e * 16) =
+                            split4(f32x4{v[4 * gg][e], v[4 * gg + 1][e], v[4 * gg + 2][e], v[4 * gg + 3][e]});
+                if (!half) *reinterpret_cast<f32x2*>(image + Image<DP>::kFrags * 1024 + d * 4) = w;   // all 16 decays
+            }
+        }
+        __syncthreads();
+        // pairs: a wave per level and product (M on the keys' waves, P on the queries'); the level of (t, j) is the
+        // highest bit of t ^ j. A lower token's row of P is some upper one's: not used.
+        if (half == 0) {
+            const int hb = (round ? 2 : 8) >> sel;
+            const uint8_t* base = lv + c16 * kRow + 16 * g;
+            const uint8_t* left = is_q ? lv + 2 * kMat + ((c16 / (2 * hb)) * hb + c16 % hb) * kRow + 16 * g : base;
+            const int dist = is_q ? kHalfMat : kMat;
+            f32x4 acc = {0, 0, 0, 0}, acc2 = {0, 0, 0, 0};
+#pragma unroll
+            for (int s = 0; s < NS; ++s) {
+                const u32x4 kh = *reinterpret_cast<const u32x4*>(base + s * 64);
+                const u32x4 kl = *reinterpret_cast<const u32x4*>(base + kMat + s * 64);
+                const u32x4 lh = *reinterpret_cast<const u32x4*>(left + s * 64);
+                const u32x4 ll = *reinterpret_cast<const u32x4*>(left + dist + s * 64);
+                acc = mfma16(lh, kh, acc);
+                acc2 = mfma16(lh, kl, acc2);
+                acc2 = mfma16(ll, kh, acc2);
+            }
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const int t = 4 * g + e, j = c16, x2 = t ^ j;
+                const float v = acc[e] + acc2[e];
+                float* dst = (is_q ? ps : ms) + t * 20 + j;
+                if (t > j && x2 >= hb && x2 < 2 * hb) *dst = is_q ? v : beta[t] * v;
+                else if (round == 0 && sel == 0 && t <= j) *dst = is_q && t == j ? diag[t] : 0.0f;
             }
         }
     }
     __syncthreads();
-    // pairs: a wave per level; the level of (t, j) is the highest bit of t ^ j
-    {
-        const int hb = 8 >> wave;
-        const uint8_t* base = mats + wave * 4 * kMat + c16 * kRow + 16 * g;
-        f32x4 dm = {0, 0, 0, 0}, dq = {0, 0, 0, 0};
+    // the level matrices are free: G K and G Q go through their place, so that the image leaves in whole pieces
+    if (sel == 1) {
 #pragma unroll
-        for (int s = 0; s < NS; ++s) {
-            const u32x4 kh = *reinterpret_cast<const u32x4*>(base + s * 64);
-            const u32x4 kl = *reinterpret_cast<const u32x4*>(base + kMat + s * 64);
-            const u32x4 qh = *reinterpret_cast<const u32x4*>(base + 2 * kMat + s * 64);
-            const u32x4 ql = *reinterpret_cast<const u32x4*>(base + 3 * kMat + s * 64);
-            dm = mfma16(kh, kh, dm);
-            dm = mfma16(kh, kl, dm);
-            dm = mfma16(kl, kh, dm);
-            dq = mfma16(qh, kh, dq);
-            dq = mfma16(qh, kl, dq);
-            dq = mfma16(ql, kh, dq);
-        }
+        for (int p = 0; p < kPer; ++p) {
+            const int d = (lane + p * 64) * 2;
+            if (d >= DP) continue;
+            f32x2 w = {1.0f, 1.0f};
+            if (half) {
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            const int t = 4 * g + e, j = c16, x = t ^ j;
-            if (t > j && x >= hb && x < 2 * hb) {
-                ms[t * 20 + j] = beta[t] * dm[e];
-                ps[t * 20 + j] = dq[e];
-            } else if (wave == 0 && t <= j) {
-                ms[t * 20 + j] = 0.0f;
-                ps[t * 20 + j] = t == j ? diag[t] : 0.0f;
+                for (int t = 0; t < 8; ++t) w = scale(w, *reinterpret_cast<const f32x2*>(lg + t * DP + d));
+            }
+#pragma unroll
+            for (int i = 0; i < 8; ++i) {
+                w = scale(w, *reinterpret_cast<const f32x2*>(lg + (r0 + i) * DP + d));
+                put(mats + (is_q ? 2 : 0) * kMat, kMat, (r0 + i) * kRow + d * 2, scale(x[p][i], w));
             }
         }
     }
     __syncthreads();
     if (wave == 0) {
         // row c16 of X = (I + M)^-1 from X (I + M) = I, last column first
-        float x[kC];
+        float y[kC];
 #pragma unroll
-        for (int j = 0; j < kC; ++j) x[j] = j == c16 ? 1.0f : 0.0f;
+        for (int j = 0; j < kC; ++j) y[j] = j == c16 ? 1.0f : 0.0f;
 #pragma unroll
         for (int s = kC - 1; s >= 1; --s) {
             float m[kC];
@@ -397,18 +454,25 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(DeltaArgs a, int chunks
                 m[j + 3] = v[3];
             }
 #pragma unroll
-            for (int j = 0; j < s; ++j) x[j] = fmaf(-x[s], m[j], x[j]);
+            for (int j = 0; j < s; ++j) y[j] = fmaf(-y[s], m[j], y[j]);
         }
         f32x4 mine = {0, 0, 0, 0};
 #pragma unroll
         for (int gg = 0; gg < 4; ++gg)
-            if (g == gg) mine = f32x4{x[4 * gg], x[4 * gg + 1], x[4 * gg + 2], x[4 * gg + 3]};
+            if (g == gg) mine = f32x4{y[4 * gg], y[4 * gg + 1], y[4 * gg + 2], y[4 * gg + 3]};
 #pragma unroll
         for (int e = 0; e < 4; ++e) mine[e] *= beta[4 * g + e];
         *reinterpret_cast<u32x4*>(image + 6 * NS * 1024 + lane * 16) = split4(mine);
-    } else if (wave == 1) {
+    } else if (wave == 4) {
         *reinterpret_cast<u32x4*>(image + (6 * NS + 1) * 1024 + lane * 16) =
             split4(*reinterpret_cast<const f32x4*>(ps + c16 * 20 + 4 * g));
+    }
+    // the other waves: fragments of matrix i / NS, step i % NS
+    if (wave == 0 || wave == 4) return;
+    for (int i = wave > 4 ? wave - 2 : wave - 1; i < 4 * NS; i += kPrepThreads / 64 - 2) {
+        const uint8_t* from = mats + (i / NS) * kMat + c16 * kRow + (i % NS) * 64 + 8 * g;
+        *reinterpret_cast<u32x4*>(image + i * 1024 + lane * 16) =
+            join(*reinterpret_cast<const u32x2*>(from), *reinterpret_cast<const u32x2*>(from + 32));
     }
 }
 
@@ -545,12 +609,12 @@ void walk_t(const DeltaArgs& a, int chunks, hipStream_t stream) {
 
 template <int DP>
 void chunk_t(const DeltaArgs& a, hipStream_t stream) {
-    constexpr int shared = 16 * kC * (DP * 2 + 16) + kC * DP * 4 + 4 * kC * 4 + 2 * kC * 20 * 4;
+    constexpr int shared = 6 * kC * (DP * 2 + 16) + kC * DP * 4 + 4 * kC * 4 + 2 * kC * 20 * 4;
     static const hipError_t once = hipFuncSetAttribute(reinterpret_cast<const void*>(&delta_prep_kernel<DP>),
                                                        hipFuncAttributeMaxDynamicSharedMemorySize, shared);
     (void)once;
     const int chunks = (a.seq + kC - 1) / kC;
-    delta_prep_kernel<DP><<<dim3((unsigned)chunks, (unsigned)a.heads, (unsigned)a.batch), 256, shared, stream>>>(a, chunks);
+    delta_prep_kernel<DP><<<dim3((unsigned)chunks, (unsigned)a.heads, (unsigned)a.batch), kPrepThreads, shared, stream>>>(a, chunks);
     // wide slices read every image once; narrow ones make more workgroups
     if (DP <= 128 && a.vp > 64 && (int64_t)a.batch * a.heads >= 256) walk_t<DP, 2>(a, chunks, stream);
     else walk_t<DP, 1>(a, chunks, stream);

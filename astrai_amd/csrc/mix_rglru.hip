@@ -26,24 +26,39 @@ struct Decay {
     float a, b;   // S <- a S + b
 };
 
-// log_a = coef r <= 0
-template <bool FAST>
-__device__ __forceinline__ Decay decay_of(float zr, float zi, float coef, float u) {
-    const float r = FAST ? sigmoid_fast(zr) : sigmoid(zr), i = FAST ? sigmoid_fast(zi) : sigmoid(zi);
-    const float log_a = coef * r;
+// log a = coef r <= 0
+__device__ __forceinline__ Decay decay_exact(float zr, float zi, float coef, float u) {
+    const float log_a = coef * sigmoid(zr);
+    return Decay{expf(log_a), sqrtf(-expm1f(2.0f * log_a)) * sigmoid(zi) * u};
+}
+
+// The same on the hardware's exponential, reciprocal and root, of sums without their biases: b = -log2(e) bias,
+// coef2 = log2(e) coef, so that e = log2 a and 1 - a^2 = 1 - 2^(2 e), a Taylor polynomial in e where the difference
+// would cancel.
+__device__ __forceinline__ Decay decay_fast(float sr, float br, float si, float bi, float coef2, float u) {
+    const float r = __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(fmaf(sr, -kLog2e, br)));
+    const float i = __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(fmaf(si, -kLog2e, bi)));
+    const float e = coef2 * r;
     Decay d;
-    if constexpr (FAST) {
-        d.a = __builtin_amdgcn_exp2f(kLog2e * log_a);
-        d.b = __builtin_amdgcn_sqrtf(one_minus_exp(2.0f * log_a, d.a * d.a)) * i * u;
-    } else {
-        d.a = expf(log_a);
-        d.b = sqrtf(-expm1f(2.0f * log_a)) * i * u;
-    }
+    d.a = __builtin_amdgcn_exp2f(e);
+    constexpr float c = 1.38629436111989061883f;   // 2 ln 2
+    float p = fmaf(e, c / 5.0f, 1.0f);
+    p = fmaf(e * (c / 4.0f), p, 1.0f);
+    p = fmaf(e * (c / 3.0f), p, 1.0f);
+    p = fmaf(e * (c / 2.0f), p, 1.0f);
+    const float m = e > -0.07f ? -c * e * p : fmaf(-d.a, d.a, 1.0f);
+    d.b = __builtin_amdgcn_sqrtf(m) * i * u;
     return d;
 }
 
+__device__ __forceinline__ float gelu_fast(float z) {   // gelu_as with log2(e) in its constants
+    constexpr float c = -kLog2e * 1.5957691216057308f;
+    const float t = z * fmaf(z * z, c * 0.044715f, c);
+    return z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(t));
+}
+
 template <int NT, bool OUT>
-__global__ __launch_bounds__(256) void rglru_chunk_kernel(RglruArgs a, int csplit) {
+__global__ __launch_bounds__(256, 3) void rglru_chunk_kernel(RglruArgs a, int csplit) {
     constexpr int kTile = NT * 16;
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
     const int bp = a.bp, row_bytes = bp * 2 + 16;
@@ -82,17 +97,49 @@ __global__ __launch_bounds__(256) void rglru_chunk_kernel(RglruArgs a, int cspli
     if (!OUT && last) return;
 
     const uint16_t* u = static_cast<const uint16_t*>(a.u) + (int64_t)b * a.seq * cols + blk * bp;
-    const int c8 = bp / 8;
+    const int c8 = bp / 8, row0 = tid / c8, e0 = tid % c8, row_step = 256 / c8, e_step = 256 % c8;
     for (int t0 = tok0; t0 < tok1; t0 += kTile) {
         __syncthreads();   // the previous tile is no longer read; the carries are there
-        for (int i = tid; i < kTile * c8; i += 256) {
-            const int t = t0 + i / c8, e = i % c8;
-            *reinterpret_cast<u32x4*>(lds + (i / c8) * row_bytes + e * 16) =
-                t < tok1 ? *reinterpret_cast<const u32x4*>(u + (int64_t)t * cols + e * 8) : u32x4{0, 0, 0, 0};
+        // (eight loads in flight; a thread's chunks are 256 apart)
+        for (int row = row0, e = e0; row < kTile;) {
+            u32x4 v[8];
+            int at[8];
+#pragma unroll
+            for (int j = 0; j < 8; ++j) {
+                at[j] = row < kTile ? row * row_bytes + e * 16 : -1;
+                const int t = t0 + row;
+                v[j] = u32x4{0, 0, 0, 0};
+                if (row < kTile && t < tok1) v[j] = *reinterpret_cast<const u32x4*>(u + (int64_t)t * cols + e * 8);
+                row += row_step;
+                e += e_step;
+                if (e >= c8) {
+                    e -= c8;
+                    ++row;
+                }
+            }
+#pragma unroll
+            for (int j = 0; j < 8; ++j)
+                if (at[j] >= 0) *reinterpret_cast<u32x4*>(lds + at[j]) = v[j];
         }
         __syncthreads();
+        const int left = min(tok1 - t0, kTile);
         for (int ct = part * 4 + wave; ct < bp / 16; ct += 4 * csplit) {
             const int ch = ct * 16 + c16, col = blk * bp + ch;
+            // the output gates' inputs, asked for ahead of the products (past the end: the last token's)
+            uint16_t yv[OUT ? NT : 1][4];
+            // (buffer descriptors end with the segment: later tokens read as 0 and are not written)
+            const __amdgpu_buffer_rsrc_t ry = w8a8::make_rsrc(
+                static_cast<const uint16_t*>(a.proj) + ((int64_t)b * a.seq + t0) * a.ld, (uint32_t)(left * a.ld) * 2);
+            const __amdgpu_buffer_rsrc_t ro = w8a8::make_rsrc(
+                static_cast<const uint16_t*>(a.out) + ((int64_t)b * a.seq + t0) * cols, (uint32_t)(left * cols) * 2);
+            const uint32_t y_lane = (uint32_t)(4 * g * a.ld + a.y_off + col) * 2, o_lane = (uint32_t)(4 * g * cols + col) * 2;
+            if constexpr (OUT) {
+#pragma unroll
+                for (int tt = 0; tt < NT; ++tt)
+#pragma unroll
+                    for (int e = 0; e < 4; ++e)
+                        yv[tt][e] = __builtin_amdgcn_raw_buffer_load_b16(ry, y_lane + (uint32_t)((tt * 16 + e) * a.ld) * 2, 0, 0);
+            }
             f32x4 zr[NT], zi[NT];
 #pragma unroll
             for (int tt = 0; tt < NT; ++tt) zr[tt] = zi[tt] = f32x4{0, 0, 0, 0};
@@ -100,9 +147,12 @@ __global__ __launch_bounds__(256) void rglru_chunk_kernel(RglruArgs a, int cspli
             const uint16_t* wr = static_cast<const uint16_t*>(a.w_r) + w_row;
             const uint16_t* wi = static_cast<const uint16_t*>(a.w_i) + w_row;
             const uint8_t* lu = lds + c16 * row_bytes + 16 * g;
+            // weight operands two steps ahead
             u32x4 fr = *reinterpret_cast<const u32x4*>(wr), fi = *reinterpret_cast<const u32x4*>(wi);
+            const int k1 = bp > 32 ? 32 : 0;
+            u32x4 mr = *reinterpret_cast<const u32x4*>(wr + k1), mi = *reinterpret_cast<const u32x4*>(wi + k1);
             for (int k = 0; k < bp; k += 32) {
-                const int kn = k + 32 < bp ? k + 32 : k;
+                const int kn = k + 64 < bp ? k + 64 : k;
                 const u32x4 nr = *reinterpret_cast<const u32x4*>(wr + kn), ni = *reinterpret_cast<const u32x4*>(wi + kn);
 #pragma unroll
                 for (int tt = 0; tt < NT; ++tt) {
@@ -110,10 +160,12 @@ __global__ __launch_bounds__(256) void rglru_chunk_kernel(RglruArgs a, int cspli
                     zr[tt] = mfma16(x, fr, zr[tt]);
                     zi[tt] = mfma16(x, fi, zi[tt]);
                 }
-                fr = nr;
-                fi = ni;
+                fr = mr;
+                fi = mi;
+                mr = nr;
+                mi = ni;
             }
-            const float br = a.b_r[col], bi = a.b_i[col], coef = a.coef[col];
+            const float br = -kLog2e * a.b_r[col], bi = -kLog2e * a.b_i[col], coef2 = kLog2e * a.coef[col];
             float s_in = carry_s[ch], a_in = carry_a[ch];
 #pragma unroll
             for (int tt = 0; tt < NT; ++tt) {
@@ -124,8 +176,15 @@ __global__ __launch_bounds__(256) void rglru_chunk_kernel(RglruArgs a, int cspli
                 for (int e = 0; e < 4; ++e) {
                     const float x = w8a8::bf16_to_f32(
                         *reinterpret_cast<const uint16_t*>(lds + (tl + e) * row_bytes + ch * 2));
-                    d[e] = decay_of<true>(zr[tt][e] + br, zi[tt][e] + bi, coef, x);
-                    if (t0 + tl + e >= tok1) d[e] = Decay{1.0f, 0.0f};
+                    d[e] = decay_fast(zr[tt][e], br, zi[tt][e], bi, coef2, x);
+                }
+                if (left < kTile) {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e)
+                        if (tl + e >= left) d[e] = Decay{1.0f, 0.0f};
+                }
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
                     pa *= d[e].a;
                     pb = fmaf(d[e].a, pb, d[e].b);
                 }
@@ -150,12 +209,8 @@ __global__ __launch_bounds__(256) void rglru_chunk_kernel(RglruArgs a, int cspli
 #pragma unroll
                     for (int e = 0; e < 4; ++e) {
                         s = fmaf(d[e].a, s, d[e].b);
-                        const int t = t0 + tl + e;
-                        if (t < tok1) {
-                            const int64_t row = (int64_t)b * a.seq + t;
-                            const float y = Elem<uint16_t>::get(static_cast<const uint16_t*>(a.proj) + row * a.ld + a.y_off + col);
-                            Elem<uint16_t>::put(static_cast<uint16_t*>(a.out) + row * cols + col, s * gelu_as<uint16_t>(y));
-                        }
+                        const float o = s * gelu_fast(w8a8::bf16_to_f32(yv[tt][e]));
+                        __builtin_amdgcn_raw_buffer_store_b16(f32_to_bf16(o), ro, o_lane + (uint32_t)((tt * 16 + e) * cols) * 2, 0, 0);
                     }
                 }
             }
@@ -225,17 +280,17 @@ __global__ __launch_bounds__(256) void rglru_step_kernel(RglruArgs a, int nb) {
     const int b = b0 + bl;
     float* state = a.state + (int64_t)b * cols + col;
     float s = *state;
-    const float coef = a.coef[col];
+    const float coef2 = kLog2e * a.coef[col];
     for (int t = 0; t < a.seq; ++t) {
         const f32x4 x4 = conv_at4<uint16_t>(a.conv, b, start, t, col & ~3);
         const int e = col & 3;
         const float x = rounded<uint16_t>(e == 0 ? x4[0] : e == 1 ? x4[1] : e == 2 ? x4[2] : x4[3]);
         const int r = bl * a.seq + t;
-        const Decay d = decay_of<true>(zs[0][r][ch], zs[1][r][ch], coef, x);
+        const Decay d = decay_fast(zs[0][r][ch], 0.0f, zs[1][r][ch], 0.0f, coef2, x);
         s = fmaf(d.a, s, d.b);
         const int64_t row = (int64_t)b * a.seq + t;
         const float y = Elem<uint16_t>::get(static_cast<const uint16_t*>(a.proj) + row * a.ld + a.y_off + col);
-        Elem<uint16_t>::put(static_cast<uint16_t*>(a.out) + row * cols + col, s * gelu_as<uint16_t>(y));
+        Elem<uint16_t>::put(static_cast<uint16_t*>(a.out) + row * cols + col, s * gelu_fast(y));
     }
     *state = s;
     // this block's last inputs into the ring: rows that no workgroup of this launch reads
@@ -259,7 +314,7 @@ __global__ __launch_bounds__(256) void rglru_gates_kernel(RglruArgs a) {
         zr = fmaf(x, Elem<T>::get(wr + (int64_t)k * a.bp), zr);
         zi = fmaf(x, Elem<T>::get(wi + (int64_t)k * a.bp), zi);
     }
-    const Decay d = decay_of<false>(zr + a.b_r[col], zi + a.b_i[col], a.coef[col], Elem<T>::get(u + ch));
+    const Decay d = decay_exact(zr + a.b_r[col], zi + a.b_i[col], a.coef[col], Elem<T>::get(u + ch));
     a.scratch[item] = d.a;
     a.scratch[tokens * cols + item] = d.b;
 }
@@ -312,10 +367,7 @@ void general_t(const RglruArgs& a, hipStream_t stream) {
 // a tile of 64 tokens of 1024 channels: 129 KiB of LDS, the carries 8 KiB
 bool rglru_chunk_supported(int bp) { return bp <= 1024; }
 
-void launch_rglru_chunk(const RglruArgs& a, hipStream_t stream) {
-    if (a.bp <= 256) chunk_t<8>(a, stream);
-    else chunk_t<4>(a, stream);
-}
+void launch_rglru_chunk(const RglruArgs& a, hipStream_t stream) { chunk_t<4>(a, stream); }
 
 bool rglru_step_supported(int bp, int seq) { return bp > 0 && seq <= kRingSteps; }
 

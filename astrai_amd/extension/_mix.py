@@ -660,7 +660,7 @@ def rglru_nseg(batch: int, blocks: int, bp: int, seq: int) -> int:
     """Segments of a sequence that run side by side: enough workgroups for one per CU, no segment shorter
     than two tiles."""
     groups = batch * blocks * -(-bp // 64)
-    tiles = -(-seq // (128 if bp <= 256 else 64))
+    tiles = -(-seq // 64)
     return max(1, min(-(-256 // groups), tiles // 2))
 
 

@@ -169,7 +169,7 @@ int astrai_mix_conv(const void* proj, int64_t ld, int64_t off, int64_t cols, con
  *   r, i = sigmoid(W u + b) per block, a = exp(coef r), S <- a S + sqrt(1 - a^2) i u, out = S gelu(y),
  * y columns of proj from y_off, b_r, b_i, coef (<= 0), state [batch, channels] float.
  * _chunk (bf16, bp <= 1024): w [blocks, out, in]; nseg segments of the sequence side by side, scratch
- * [batch, nseg, 2, channels] float when nseg > 1; a segment has tiles of 128 tokens (64 with bp > 256).
+ * [batch, nseg, 2, channels] float when nseg > 1; a segment is a whole number of tiles of 64 tokens.
  * _general (bf16 or float): w [blocks, in, out], scratch [2, batch * seq, channels].
  * _step (bf16, seq <= RING_STEPS): convolves proj's columns from x_off itself and updates the ring (as above). */
 int astrai_mix_rglru_chunk(const void* u, const void* proj, int64_t ld, int64_t y_off, const void* w_r, const void* w_i,
