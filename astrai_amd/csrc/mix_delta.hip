@@ -37,7 +37,7 @@ constexpr int kStepThreads = 512, kStepWaves = kStepThreads / 64;
 
 // thread (rg, vq): value columns 4 vq .., state rows rg + RG i; vq runs over vqp = a power of two >= vp / 4
 template <typename T, int NR, bool FUSED>
-__global__ __launch_bounds__(kStepThreads) void delta_step_kernel(DeltaArgs a, int vqp) {
+__global__ __launch_bounds__(kStepThreads, NR <= 8 ? 4 : 2) void delta_step_kernel(DeltaArgs a, int vqp) {
     extern __shared__ __attribute__((aligned(16))) float sh[];
     const int rgs = kStepThreads / vqp, rows = rgs * NR;   // rows >= dp, those past it zero
     float* const qs = sh;                   // [rows]
@@ -131,7 +131,7 @@ __global__ __launch_bounds__(kStepThreads) void delta_step_kernel(DeltaArgs a, i
         __syncthreads();
         f32x4 o = {0, 0, 0, 0}, u = {0, 0, 0, 0};
         kq = 0.0f;
-#pragma unroll
+#pragma unroll 2
         for (int w = 0; w < kStepWaves; ++w) {
             u += *reinterpret_cast<const f32x4*>(red + (w * vqp + vq) * 4);
             o += *reinterpret_cast<const f32x4*>(red + ((kStepWaves + w) * vqp + vq) * 4);

@@ -238,23 +238,38 @@ __global__ __launch_bounds__(256, 3) void rglru_chunk_kernel(RglruArgs a, int cs
 __global__ __launch_bounds__(256) void rglru_step_kernel(RglruArgs a, int nb) {
     __shared__ f32x4 red[3][2][64];
     __shared__ float zs[2][16][17];
+    __shared__ float us[16][17];   // the convolved inputs of this workgroup's channels
     const int tid = threadIdx.x, lane = tid & 63, c16 = lane & 15, g = lane >> 4;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int bp = a.bp, per = bp / 16, cols = a.blocks * bp;
     const int blk = (int)blockIdx.x / per, ct = (int)blockIdx.x % per;
-    const int b0 = (int)blockIdx.y * nb, nlive = min(nb, a.batch - b0) * a.seq;
+    const int b0 = (int)blockIdx.y * nb, n_seq = min(nb, a.batch - b0), n_live = n_seq * a.seq;
     const int64_t start = a.conv.positions[0];
+    // for the recurrence a thread takes one channel of one sequence; what it needs is asked for now
+    const int ch = tid & 15, col = blk * bp + ct * 16 + ch, bl = tid >> 4;
+    const bool mine = bl < n_seq;
+    const int b = b0 + (mine ? bl : 0);
+    const uint16_t* y_src = static_cast<const uint16_t*>(a.proj) + (int64_t)b * a.seq * a.ld + a.y_off + col;
+    float s = a.state[(int64_t)b * cols + col];
+    const float coef2 = kLog2e * a.coef[col], br = -kLog2e * a.b_r[col], bi = -kLog2e * a.b_i[col];
+    uint16_t y_next = y_src[0];
     {
-        const int row = min(c16, nlive - 1), b = b0 + row / a.seq, t = row % a.seq;
+        const int row = min(c16, n_live - 1), rb = b0 + row / a.seq, t = row % a.seq;
         const int64_t w_row = ((int64_t)blk * bp + ct * 16 + c16) * bp;
         f32x4 zr = {0, 0, 0, 0}, zi = {0, 0, 0, 0};
         for (int k = wave * 32 + 8 * g; k < bp; k += 128) {
             const u32x4 fr = *reinterpret_cast<const u32x4*>(static_cast<const uint16_t*>(a.w_r) + w_row + k);
             const u32x4 fi = *reinterpret_cast<const u32x4*>(static_cast<const uint16_t*>(a.w_i) + w_row + k);
-            const f32x4 x0 = conv_at4<uint16_t>(a.conv, b, start, t, blk * bp + k);
-            const f32x4 x1 = conv_at4<uint16_t>(a.conv, b, start, t, blk * bp + k + 4);
+            const f32x4 x0 = conv_at4<uint16_t>(a.conv, rb, start, t, blk * bp + k);
+            const f32x4 x1 = conv_at4<uint16_t>(a.conv, rb, start, t, blk * bp + k + 4);
             const u32x4 x = {pack_bf16x2(x0[0], x0[1]), pack_bf16x2(x0[2], x0[3]), pack_bf16x2(x1[0], x1[1]),
                              pack_bf16x2(x1[2], x1[3])};
+            if (k / 16 == ct) {
+                float f[8];
+                w8a8::unpack8(x, f);
+#pragma unroll
+                for (int e = 0; e < 8; ++e) us[c16][k % 16 + e] = f[e];
+            }
             zr = mfma16(x, fr, zr);
             zi = mfma16(x, fi, zi);
         }
@@ -264,35 +279,24 @@ __global__ __launch_bounds__(256) void rglru_step_kernel(RglruArgs a, int nb) {
         }
         __syncthreads();
         if (wave == 0) {
-            const int col = blk * bp + ct * 16 + c16;
-            const float br = a.b_r[col], bi = a.b_i[col];
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
-                zs[0][4 * g + e][c16] = ((zr[e] + red[0][0][lane][e]) + (red[1][0][lane][e] + red[2][0][lane][e])) + br;
-                zs[1][4 * g + e][c16] = ((zi[e] + red[0][1][lane][e]) + (red[1][1][lane][e] + red[2][1][lane][e])) + bi;
+                zs[0][4 * g + e][c16] = (zr[e] + red[0][0][lane][e]) + (red[1][0][lane][e] + red[2][0][lane][e]);
+                zs[1][4 * g + e][c16] = (zi[e] + red[0][1][lane][e]) + (red[1][1][lane][e] + red[2][1][lane][e]);
             }
         }
         __syncthreads();
     }
-    // a thread: one channel of one sequence
-    const int ch = tid & 15, col = blk * bp + ct * 16 + ch, bl = tid >> 4;
-    if (bl >= min(nb, a.batch - b0)) return;
-    const int b = b0 + bl;
-    float* state = a.state + (int64_t)b * cols + col;
-    float s = *state;
-    const float coef2 = kLog2e * a.coef[col];
+    if (!mine) return;
     for (int t = 0; t < a.seq; ++t) {
-        const f32x4 x4 = conv_at4<uint16_t>(a.conv, b, start, t, col & ~3);
-        const int e = col & 3;
-        const float x = rounded<uint16_t>(e == 0 ? x4[0] : e == 1 ? x4[1] : e == 2 ? x4[2] : x4[3]);
         const int r = bl * a.seq + t;
-        const Decay d = decay_fast(zs[0][r][ch], 0.0f, zs[1][r][ch], 0.0f, coef2, x);
+        const float y = w8a8::bf16_to_f32(y_next);
+        if (t + 1 < a.seq) y_next = y_src[(int64_t)(t + 1) * a.ld];
+        const Decay d = decay_fast(zs[0][r][ch], br, zs[1][r][ch], bi, coef2, us[r][ch]);
         s = fmaf(d.a, s, d.b);
-        const int64_t row = (int64_t)b * a.seq + t;
-        const float y = Elem<uint16_t>::get(static_cast<const uint16_t*>(a.proj) + row * a.ld + a.y_off + col);
-        Elem<uint16_t>::put(static_cast<uint16_t*>(a.out) + row * cols + col, s * gelu_fast(y));
+        Elem<uint16_t>::put(static_cast<uint16_t*>(a.out) + ((int64_t)b * a.seq + t) * cols + col, s * gelu_fast(y));
     }
-    *state = s;
+    a.state[(int64_t)b * cols + col] = s;
     // this block's last inputs into the ring: rows that no workgroup of this launch reads
     if (ch % 4 == 0)
         for (int t = max(a.seq - a.conv.taps + 1, 0); t < a.seq; ++t) ring_put4<uint16_t>(a.conv, b, start, t, col);
