@@ -518,11 +518,23 @@ __global__ __launch_bounds__(256, DP <= 128 ? 2 : 1) void delta_walk_kernel(Delt
                 vr[vt][e] = (t < a.seq && v < a.vp) ? vsrc[(int64_t)t * a.ldq + v] : 0;
             }
     };
+    f32x4 o[VT];
+    auto put_o = [&](int c) {
+#pragma unroll
+        for (int vt = 0; vt < VT; ++vt)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const int t = c * kC + 4 * g + e, v = v0 + 16 * vt + c16;
+                if (t < a.seq && v < a.vp)
+                    Elem<uint16_t>::put(static_cast<uint16_t*>(a.out) + (((int64_t)b * a.seq + t) * a.heads + h) * a.vp + v, o[vt][e]);
+            }
+    };
     dma(0);
     fetch_v(0);
     for (int c = 0; c < chunks; ++c) {
         __builtin_amdgcn_s_waitcnt(0x0070);   // vmcnt(0) lgkmcnt(0)
         __syncthreads();                      // image c is there, image c - 1 is no longer read
+        if (c) put_o(c - 1);                  // (stores count as outstanding memory operations too: early in the chunk)
         dma(c + 1);
         f32x4 x[VT];
 #pragma unroll
@@ -532,7 +544,7 @@ __global__ __launch_bounds__(256, DP <= 128 ? 2 : 1) void delta_walk_kernel(Delt
         fetch_v(c + 1);
         const uint8_t* im = lds + (c & 1) * kBuf;
         auto frag = [&](int i) { return *reinterpret_cast<const u32x4*>(im + i * 1024 + lane * 16); };
-        f32x4 y[VT], o[VT];
+        f32x4 y[VT];
 #pragma unroll
         for (int vt = 0; vt < VT; ++vt) y[vt] = o[vt] = f32x4{0, 0, 0, 0};
 #pragma unroll
@@ -577,15 +589,8 @@ __global__ __launch_bounds__(256, DP <= 128 ? 2 : 1) void delta_walk_kernel(Delt
                 st[i][vt] = mfma16(kf, ul[vt], st[i][vt]);
             }
         }
-#pragma unroll
-        for (int vt = 0; vt < VT; ++vt)
-#pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                const int t = c * kC + 4 * g + e, v = v0 + 16 * vt + c16;
-                if (t < a.seq && v < a.vp)
-                    Elem<uint16_t>::put(static_cast<uint16_t*>(a.out) + (((int64_t)b * a.seq + t) * a.heads + h) * a.vp + v, o[vt][e]);
-            }
     }
+    put_o(chunks - 1);
 #pragma unroll
     for (int i = 0; i < NT; ++i)
 #pragma unroll
